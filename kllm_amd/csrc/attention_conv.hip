@@ -1,6 +1,7 @@
 // What lies between the query/key/value product and attention for a mixer whose three projections
-// pass a short causal convolution per channel: convolution, rotation of the first `rot` elements of
-// every query and key head, queries out, keys and values into pages.  All in 32-bit.
+// pass a short causal convolution per channel, or have biases, or are to be padded: convolution (none
+// without its weights), bias, rotation of the first `rot` elements of every query and key head,
+// queries out, keys and values into pages (queries alone without a cache: KV is 0).  All in 32-bit.
 //
 // A wave takes a tile of tokens (16, or one in a step of single tokens) and one head of q, k or v:
 // the tile's rows and the taps - 1 rows before it pass through LDS once (the sums' slices added on the
@@ -29,7 +30,7 @@ __global__ __launch_bounds__(64 * kConvWaves) void qkv_conv_append_kernel(
     T* __restrict__ cache, const int* __restrict__ positions, const int* __restrict__ span_of_token,
     const int* __restrict__ slots, const int* __restrict__ span_start, const int* __restrict__ span_pos,
     const int* __restrict__ block_table, int max_pages, int page_size, int n, int H, int KV, int dk, int dv, int width,
-    int ld) {
+    int ld, const float* __restrict__ bias) {
   extern __shared__ float conv_lds[];                  // [waves][TILE + taps - 1][ld]
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   const int item = blockIdx.y * kConvWaves + wave;
@@ -44,17 +45,18 @@ __global__ __launch_bounds__(64 * kConvWaves) void qkv_conv_append_kernel(
   // lane l looks up where token l % TILE of the tile goes, before anything waits
   const long my_t = first + min(lane % TILE, nt - 1);
   const int my_pos = positions[my_t];
-  const int my_page = block_table[(long)span_of_token[my_t] * max_pages + my_pos / page_size];
+  const int my_page = cache ? block_table[(long)span_of_token[my_t] * max_pages + my_pos / page_size] : 0;
   const int my_slot = my_pos % page_size;
   if (there) {
     // rows before the tile may belong to other requests: then they are not looked at.  Eight rows' loads
     // go out together.
     for (int e = lane; e < len; e += kWave) {
       const float* src = in + ch0 + e;
+      const float b = bias ? bias[ch0 + e] : 0.f;
       for (int r0 = 0; r0 < K + nt; r0 += 8) {
         float v[8];
 #pragma unroll
-        for (int u = 0; u < 8; ++u) v[u] = 0.f;
+        for (int u = 0; u < 8; ++u) v[u] = b;
         for (int sl = 0; sl < nsplit; ++sl)
 #pragma unroll
           for (int u = 0; u < 8; ++u) {
@@ -72,7 +74,7 @@ __global__ __launch_bounds__(64 * kConvWaves) void qkv_conv_append_kernel(
   // other tile asks token by token where each input is.
   const int span_first = span_of_token[first];
   const bool inside = span_of_token[first + nt - 1] == span_first && first - K >= span_start[span_first];
-  if (there) {
+  if (there && conv_w) {
     for (int e = lane; e < len; e += kWave) {
       const float* w = conv_w + (long)(ch0 + e) * taps;
       float y[TILE];
@@ -176,10 +178,11 @@ extern "C" int kllm_qkv_conv_append(const float* sums, int nsplit, long split_st
                                     void* q_out, void* cache, const int* positions, const int* span_of_token,
                                     const int* slots, const int* span_start, const int* span_pos,
                                     const int* block_table, int max_pages, int page_size, int n, int H, int KV, int dk,
-                                    int dv, int width, int dtype, hipStream_t stream) {
-  KLLM_REQUIRE(sums && conv_w && q_out && cache && positions && span_of_token && slots && span_start && span_pos &&
-                   block_table, "qkv_conv_append: null pointer");
-  KLLM_REQUIRE(n > 0 && H > 0 && KV > 0 && dk > 0 && dv > 0 && dk <= width && dv <= width && nsplit >= 1 && col0 >= 0 &&
+                                    int dv, int width, int dtype, const float* bias, hipStream_t stream) {
+  KLLM_REQUIRE(sums && q_out && positions && span_of_token && slots && span_start && span_pos && block_table,
+               "qkv_conv_append: null pointer");
+  KLLM_REQUIRE((conv_w || taps == 1) && (!conv_w || !bias), "qkv_conv_append: a convolution has weights and no bias in front of it");
+  KLLM_REQUIRE(n > 0 && H > 0 && (cache ? KV > 0 : KV == 0) && dk > 0 && dv > 0 && dk <= width && dv <= width && nsplit >= 1 && col0 >= 0 &&
                    col0 + (H + KV) * dk + KV * dv <= row_len,
                "qkv_conv_append: bad sizes n=%d H=%d KV=%d dk=%d dv=%d width=%d row=%d", n, H, KV, dk, dv, width, row_len);
   KLLM_REQUIRE(taps >= 1 && taps <= kMaxTaps && (taps == 1 || state), "qkv_conv_append: %d taps (1 to %d), with their state",
@@ -200,7 +203,7 @@ extern "C" int kllm_qkv_conv_append(const float* sums, int nsplit, long split_st
     hipLaunchKernelGGL((qkv_conv_append_kernel<T, TILE>), grid, dim3(64 * kConvWaves), lds, stream, sums + col0, nsplit, \
                        split_stride, (long)row_len, conv_w, taps, state, slot_stride, single && taps > 1 ? 1 : 0, cos_t, sin_t, \
                        rot, interleaved, v_scale, (T*)q_out, (T*)cache, positions, span_of_token, slots, span_start,   \
-                       span_pos, block_table, max_pages, page_size, n, H, KV, dk, dv, width, ld);                      \
+                       span_pos, block_table, max_pages, page_size, n, H, KV, dk, dv, width, ld, bias);                \
   } while (0)
   if (dtype == DT_F32) {
     if (single) KLLM_QC(float, 1); else KLLM_QC(float, kConvTile);

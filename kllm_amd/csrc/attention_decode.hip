@@ -59,8 +59,9 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void attn_decode_mfma_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ final_out, float* __restrict__ part,
     const bf16_t* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ span_of_token,
-    const int* __restrict__ block_table, int max_pages, int page_size, int H, int KV, int window, int chunk, int sink,
-    int keep_first, float scale, const float* __restrict__ slopes, int head_tiles, const int* __restrict__ token_list) {
+    const int* __restrict__ block_table, int max_pages, int page_size, int H, int KV, int window, int chunk,
+    const float* __restrict__ sinks, int keep_first, float scale, const float* __restrict__ slopes, int head_tiles,
+    const int* __restrict__ token_list, const OutGate gate) {
   constexpr int hd = 16 * HDT;
   constexpr int KS = (hd + 31) / 32;           // MFMA steps over head_dim for the scores
   constexpr int kDecodeAhead = decode_ahead(HDT);
@@ -100,10 +101,10 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void attn_decode_mfma_kernel(
                  : zero8;
   }
 
-  // A sink (a key whose score is 0 and that has no value) is where the running maximum and
-  // sum of the first slice start: one of the four lanes of a column holds its exp(0).
-  const bool owns_sink = sink && slice == 0;
-  float m = owns_sink ? 0.f : -INFINITY, l = (owns_sink && g == 0) ? 1.f : 0.f;
+  // A sink (a key with a score of its own and no value) is where the running maximum and
+  // sum of the first slice start: one of the four lanes of a column holds its term, 1.
+  const bool owns_sink = sinks && slice == 0;
+  float m = owns_sink ? sinks[head] : -INFINITY, l = (owns_sink && g == 0) ? 1.f : 0.f;
   floatx4 acc[HDT];
 #pragma unroll
   for (int i = 0; i < HDT; ++i) acc[i] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -282,9 +283,10 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void attn_decode_mfma_kernel(
     const int head_o = kvh * G + ht * 16 + hc;
     if (whole) {
       const float inv = 1.f / L;
+      const floatx4 og = out_gate4(gate, t, head_o, d4);
       bf16x4 o;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] = (bf16_t)(v[i] * inv);
+      for (int i = 0; i < 4; ++i) o[i] = (bf16_t)(v[i] * inv * og[i]);
       *reinterpret_cast<bf16x4*>(final_out + ((long)t * H + head_o) * hd + d4) = o;
     } else {
       float* out = part + (((long)t * H + head_o) * gridDim.z + blockIdx.z) * (hd + 2);   // 8-byte rows
@@ -298,8 +300,9 @@ __global__ __launch_bounds__(64 * kDecodeWaves) void attn_decode_mfma_kernel(
 template <int HDT, int W>
 static int launch_decode(dim3 grid, hipStream_t stream, const void* q, void* out, float* part,
                          const void* cache, const int* positions, const int* span_of_token,
-                         const int* block_table, int max_pages, int page_size, int H, int KV, int window, int chunk, int sink,
-                         int keep_first, float scale, const float* slopes, int head_tiles, const int* token_list) {
+                         const int* block_table, int max_pages, int page_size, int H, int KV, int window, int chunk,
+                         const float* sinks, int keep_first, float scale, const float* slopes, int head_tiles,
+                         const int* token_list, const OutGate& gate) {
   const int heads = H / KV < 16 ? H / KV : 16;
   const size_t lds = (size_t)W * heads * (16 * HDT + 4) * sizeof(float);
   static int raised = 0;
@@ -321,7 +324,7 @@ static int launch_decode(dim3 grid, hipStream_t stream, const void* q, void* out
     }
     hipLaunchKernelGGL((attn_decode_mfma_kernel<HDT, W, true>), grid, dim3(64 * W), lds, stream,
                        (const bf16_t*)q, (bf16_t*)out, part, (const bf16_t*)cache, positions, span_of_token,
-                       block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes, head_tiles, token_list);
+                       block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes, head_tiles, token_list, gate);
     return 0;
   }
   if (keep_first > 0) {
@@ -335,12 +338,12 @@ static int launch_decode(dim3 grid, hipStream_t stream, const void* q, void* out
     }
     hipLaunchKernelGGL((attn_decode_mfma_kernel<HDT, W, false, true>), grid, dim3(64 * W), lds, stream,
                        (const bf16_t*)q, (bf16_t*)out, part, (const bf16_t*)cache, positions, span_of_token,
-                       block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes, head_tiles, token_list);
+                       block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes, head_tiles, token_list, gate);
     return 0;
   }
   hipLaunchKernelGGL((attn_decode_mfma_kernel<HDT, W>), grid, dim3(64 * W), lds, stream,
                      (const bf16_t*)q, (bf16_t*)out, part, (const bf16_t*)cache, positions, span_of_token,
-                     block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes, head_tiles, token_list);
+                     block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes, head_tiles, token_list, gate);
   return 0;
 }
 
@@ -437,8 +440,10 @@ extern "C" int kllm_attn_decode_slices(int n, int KV, int H, int hd, int dtype, 
 static int attn_decode_run(const char* who, const void* q, void* out, float* part, long part_floats,
                            const void* cache, const int* positions, const int* span_of_token,
                            const int* block_table, int max_pages, int page_size, int n, int H, int KV,
-                           int hd, int window, int chunk, int sink, int keep_first, float scale, const float* slopes, int nslices, int dtype,
-                           const int* token_list, int n_listed, hipStream_t stream) {
+                           int hd, int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes, int nslices,
+                           int dtype, const int* token_list, int n_listed, const OutGate& gate, hipStream_t stream) {
+  KLLM_REQUIRE(!gate.sums || (gate.nsplit >= 1 && gate.width > 0 && gate.width <= hd && gate.row >= (long)H * gate.width),
+               "%s: a gate of %d columns a head for heads of %d, rows of %ld", who, gate.width, hd, gate.row);
   KLLM_REQUIRE(q && out && part && cache && positions && span_of_token && block_table,
                "%s: null pointer", who);
   KLLM_REQUIRE(dtype == DT_BF16 || dtype == DT_F32, "%s: unknown dtype %d", who, dtype);
@@ -454,8 +459,8 @@ static int attn_decode_run(const char* who, const void* q, void* out, float* par
     KLLM_REQUIRE(H <= 65535, "%s: too many heads for the grid", who);
     KLLM_REQUIRE(!token_list || (n_listed > 0 && n_listed <= n), "%s: bad token list", who);
     return attn_f32_decode((const float*)q, (float*)out, part, (const float*)cache, positions, span_of_token,
-                           block_table, max_pages, page_size, H, KV, hd, window, chunk, sink, scale, slopes, nslices, token_list,
-                           token_list ? n_listed : n, stream);
+                           block_table, max_pages, page_size, H, KV, hd, window, chunk, sinks, scale, slopes, nslices, token_list,
+                           token_list ? n_listed : n, gate, stream);
   }
   KLLM_REQUIRE(hd % 16 == 0 && hd >= 16 && hd <= 256 && (hd <= 128 || hd == 192 || hd == 256),
                "%s: head_dim %d is not built (16..128 in steps of 16, 192, 256)", who, hd);
@@ -479,12 +484,12 @@ static int attn_decode_run(const char* who, const void* q, void* out, float* par
     if (int rc = nslices == 1                                                                     \
                      ? launch_decode<HDT, decode_waves_whole(HDT)>(                               \
                            grid, stream, q, out, part, cache, positions, span_of_token,           \
-                           block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes,          \
-                           head_tiles, token_list)                                                            \
+                           block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes,         \
+                           head_tiles, token_list, gate)                                                            \
                      : launch_decode<HDT, kDecodeWavesShared>(                                    \
                            grid, stream, q, out, part, cache, positions, span_of_token,           \
-                           block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes,          \
-                           head_tiles, token_list))                                                           \
+                           block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes,         \
+                           head_tiles, token_list, gate))                                                           \
       return rc;                                                                                  \
     break
   switch (hd / 16) {
@@ -495,7 +500,7 @@ static int attn_decode_run(const char* who, const void* q, void* out, float* par
 #undef KLLM_DEC
   KLLM_CHECK_LAUNCH(who);
   if (nslices == 1) return 0;                      // the one workgroup of a token has written the output
-  launch_attn_merge<bf16_t>((bf16_t*)out, part, count, H, hd, nslices, token_list, stream);
+  launch_attn_merge<bf16_t>((bf16_t*)out, part, count, H, hd, nslices, token_list, gate, stream);
   KLLM_CHECK_LAUNCH("attn_merge");
   return 0;
 }
@@ -503,11 +508,13 @@ static int attn_decode_run(const char* who, const void* q, void* out, float* par
 extern "C" int kllm_attn_decode(const void* q, void* out, float* part, long part_floats,
                                 const void* cache, const int* positions, const int* span_of_token,
                                 const int* block_table, int max_pages, int page_size, int n, int H,
-                                int KV, int hd, int window, int chunk, int sink, int keep_first, float scale, const float* slopes, int nslices, int dtype,
-                                const int* token_list, int n_listed, hipStream_t stream) {
+                                int KV, int hd, int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes,
+                                int nslices, int dtype, const int* token_list, int n_listed, const float* gate_sums,
+                                int gate_nsplit, long gate_stride, long gate_row, int gate_width, hipStream_t stream) {
+  const OutGate gate = {gate_sums, gate_nsplit, gate_width, gate_stride, gate_row};
   return attn_decode_run("attn_decode", q, out, part, part_floats, cache, positions, span_of_token,
-                         block_table, max_pages, page_size, n, H, KV, hd, window, chunk, sink, keep_first, scale, slopes, nslices, dtype,
-                         token_list, n_listed, stream);
+                         block_table, max_pages, page_size, n, H, KV, hd, window, chunk, sinks, keep_first, scale, slopes, nslices, dtype,
+                         token_list, n_listed, gate, stream);
 }
 
 // ---- the entry point that allocates nothing -------------------------------------------------
@@ -573,6 +580,6 @@ extern "C" int kllm_attn_decode_static(const void* q, void* out, const void* cac
   // Nothing in the scratch has to start at zero: the first kernel writes every partial result
   // (maximum, sum, output of each token, head and slice) that the second one reads.
   return attn_decode_run("attn_decode_static", q, out, part, (long)KLLM_ATTN_DECODE_STATIC_FLOATS, cache,
-                         positions, span_of_token, block_table, max_pages, page_size, n, H, KV, hd, window, 0, 0, 0,
-                         scale, nullptr, nslices, dtype, token_list, n_listed, stream);
+                         positions, span_of_token, block_table, max_pages, page_size, n, H, KV, hd, window, 0, nullptr, 0,
+                         scale, nullptr, nslices, dtype, token_list, n_listed, OutGate{}, stream);
 }

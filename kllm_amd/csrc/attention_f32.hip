@@ -60,7 +60,9 @@ struct AttnF32Args {
   const int* block_table;
   int count;                   // decode: tokens; prompt: blocks of 128
   int max_pages, page_size, H, KV, hd, window;
-  int chunk, sink;             // a chunked mask (0: none); a key whose score is 0 and that has no value
+  int chunk;                   // a chunked mask (0: none)
+  const float* sinks;          // per head: the score of one more key that has no value (null: none)
+  OutGate gate;                // on the output (none: no sums)
   float scale;
   const float* slopes;         // per head: a bias that grows with the distance to the key (null: none)
   int nslices, col_blocks;     // decode: slices of the keys, blocks of 32 heads per group
@@ -168,9 +170,9 @@ __global__ __launch_bounds__(64 * kF32Waves) void attn_f32_mfma_kernel(const Att
   const long page_stride = 2L * KV * block;
 
   // A sink is where the running maximum and sum of the first slice start; one of a column's
-  // two lanes holds its exp(0).
-  const bool owns_sink = a.sink && slice == 0;
-  float m = owns_sink ? 0.f : -INFINITY, l = (owns_sink && g == 0) ? 1.f : 0.f;
+  // two lanes holds its term, 1.
+  const bool owns_sink = a.sinks && slice == 0;
+  float m = owns_sink ? a.sinks[my_head] : -INFINITY, l = (owns_sink && g == 0) ? 1.f : 0.f;
   floatx16 acc[HDT];
 #pragma unroll
   for (int r = 0; r < HDT; ++r)
@@ -356,9 +358,10 @@ __global__ __launch_bounds__(64 * kF32Waves) void attn_f32_mfma_kernel(const Att
       for (int b = 0; b < 4; ++b) {
         const int d = 32 * r + 8 * b + 4 * g;
         if (d < hd) {
+          const floatx4 og = out_gate4(a.gate, my_tok, my_head, d);
           floatx4 v;
 #pragma unroll
-          for (int j = 0; j < 4; ++j) v[j] = acc[r][4 * b + j] * inv;
+          for (int j = 0; j < 4; ++j) v[j] = acc[r][4 * b + j] * inv * og[j];
           *reinterpret_cast<floatx4*>(orow + d) = v;
         }
       }
@@ -433,8 +436,8 @@ int attn_f32_slices(int n, int KV, int H, int max_keys) {
 
 int attn_f32_decode(const float* q, float* out, float* part, const float* cache, const int* positions,
                     const int* span_of_token, const int* block_table, int max_pages, int page_size,
-                    int H, int KV, int hd, int window, int chunk, int sink, float scale, const float* slopes, int nslices, const int* token_list,
-                    int count, hipStream_t stream) {
+                    int H, int KV, int hd, int window, int chunk, const float* sinks, float scale, const float* slopes, int nslices,
+                    const int* token_list, int count, const OutGate& gate, hipStream_t stream) {
   KLLM_REQUIRE(attn_f32_fits(hd, page_size),
                "attn_decode float32: head_dim %d must be a multiple of 8 up to 256 and page_size %d a multiple of 4",
                hd, page_size);
@@ -444,14 +447,14 @@ int attn_f32_decode(const float* q, float* out, float* part, const float* cache,
   a.q = q; a.out = out; a.part = part; a.cache = cache;
   a.positions = positions; a.span_of_token = span_of_token; a.token_list = token_list;
   a.block_table = block_table; a.count = count;
-  a.max_pages = max_pages; a.page_size = page_size; a.H = H; a.KV = KV; a.hd = hd; a.window = window; a.chunk = chunk; a.sink = sink;
+  a.max_pages = max_pages; a.page_size = page_size; a.H = H; a.KV = KV; a.hd = hd; a.window = window; a.chunk = chunk; a.sinks = sinks; a.gate = gate;
   a.scale = scale; a.slopes = slopes; a.nslices = nslices; a.col_blocks = (H / KV + 31) / 32;
   a.wg_merge = nslices % kF32Waves == 0;
   const long items = (long)count * KV * a.col_blocks * nslices;
   if (int rc = dispatch_f32<true>(a, items, stream)) return rc;
   KLLM_CHECK_LAUNCH("attn_decode float32");
   if (nslices > 1) {
-    launch_attn_merge<float>(out, part, count, H, hd, a.wg_merge ? nslices / kF32Waves : nslices, token_list, stream);
+    launch_attn_merge<float>(out, part, count, H, hd, a.wg_merge ? nslices / kF32Waves : nslices, token_list, gate, stream);
     KLLM_CHECK_LAUNCH("attn_merge float32");
   }
   return 0;
@@ -459,7 +462,8 @@ int attn_f32_decode(const float* q, float* out, float* part, const float* cache,
 
 int attn_f32_prefill(const float* q, float* out, const float* cache, const int* query_tiles, int n_tiles,
                      const int* span_start, const int* span_pos, const int* block_table, int max_pages,
-                     int page_size, int H, int KV, int hd, int window, int chunk, int sink, float scale, const float* slopes, hipStream_t stream) {
+                     int page_size, int H, int KV, int hd, int window, int chunk, const float* sinks, float scale, const float* slopes,
+                     const OutGate& gate, hipStream_t stream) {
   KLLM_REQUIRE(attn_f32_fits(hd, page_size),
                "attn_prefill float32: head_dim %d must be a multiple of 8 up to 256 and page_size %d a multiple of 4",
                hd, page_size);
@@ -467,7 +471,7 @@ int attn_f32_prefill(const float* q, float* out, const float* cache, const int* 
   a.q = q; a.out = out; a.cache = cache;
   a.query_tiles = query_tiles; a.span_start = span_start; a.span_pos = span_pos;
   a.block_table = block_table; a.count = n_tiles;
-  a.max_pages = max_pages; a.page_size = page_size; a.H = H; a.KV = KV; a.hd = hd; a.window = window; a.chunk = chunk; a.sink = sink;
+  a.max_pages = max_pages; a.page_size = page_size; a.H = H; a.KV = KV; a.hd = hd; a.window = window; a.chunk = chunk; a.sinks = sinks; a.gate = gate;
   a.scale = scale; a.slopes = slopes; a.nslices = 1; a.col_blocks = 1;
   const long items = (long)n_tiles * 4 * H;
   if (int rc = dispatch_f32<false>(a, items, stream)) return rc;

@@ -12,8 +12,9 @@
 // Options that a design may ask for: values of another width than the keys
 // (vd); a chunked mask (chunk > 0: the query at p reads no key before
 // p - p % chunk, chunks counted from position 0 of the request); a sink
-// (sink != 0: the softmax's denominator has one more term, exp(0), a key whose
-// score is 0 and whose value is nothing); kept first positions (keep_first > 0: the first
+// (sinks: the softmax's denominator of head h has one more term, exp(sinks[h]), a key
+// with that score and no value, neither scaled nor biased); a gate on the output (OutGate);
+// kept first positions (keep_first > 0: the first
 // keep_first positions of a request stay readable behind the window, at their true places).
 //
 // Page layout: keys [KV][slot][hd], then values [KV][vd][slot].
@@ -32,7 +33,8 @@ __global__ __launch_bounds__(kAttnThreads) void attn_generic_kernel(
     const T* __restrict__ q, T* __restrict__ out, const T* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ span_of_token,
     const int* __restrict__ block_table, int max_pages, int page_size, int H, int KV, int hd,
-    int vd, int window, int chunk, int sink, float scale, const float* __restrict__ slopes, int keep_first) {
+    int vd, int window, int chunk, const float* __restrict__ sinks, float scale, const float* __restrict__ slopes,
+    int keep_first, const OutGate gate) {
   __shared__ float qs[kMaxHeadDim];
   __shared__ float ps[kAttnThreads];
   __shared__ float red[16];
@@ -103,10 +105,10 @@ __global__ __launch_bounds__(kAttnThreads) void attn_generic_kernel(
   }
   }
 
-  if (sink) {   // one more key whose score is 0: it joins the sum, and nothing else
-    const float m_all = fmaxf(m, 0.f);
+  if (sinks) {   // one more key: it joins the sum, and nothing else
+    const float sink = sinks[h], m_all = fmaxf(m, sink);
     const float alpha = expf(m - m_all);
-    l = l * alpha + expf(-m_all);
+    l = l * alpha + expf(sink - m_all);
     acc *= alpha;
   }
   part[tid] = pv_thread ? acc : 0.f;
@@ -114,7 +116,7 @@ __global__ __launch_bounds__(kAttnThreads) void attn_generic_kernel(
   if (tid < vd) {
     float o = 0.f;
     for (int s2 = 0; s2 < nslice; ++s2) o += part[s2 * vd + tid];
-    out[((long)t * H + h) * vd + tid] = from_f32<T>(o / l);
+    out[((long)t * H + h) * vd + tid] = from_f32<T>(o / l * out_gate(gate, t, h, tid));
   }
 }
 
@@ -125,8 +127,12 @@ using namespace kllm;
 extern "C" int kllm_attn_generic(const void* q, void* out, const void* cache, const int* positions,
                                  const int* span_of_token, const int* block_table, int max_pages,
                                  int page_size, int n, int H, int KV, int hd, int vd, int window,
-                                 int chunk, int sink, float scale, const float* slopes, int dtype,
-                                 int keep_first, hipStream_t stream) {
+                                 int chunk, const float* sinks, float scale, const float* slopes, int dtype,
+                                 int keep_first, const float* gate_sums, int gate_nsplit, long gate_stride,
+                                 long gate_row, int gate_width, hipStream_t stream) {
+  const OutGate gate = {gate_sums, gate_nsplit, gate_width, gate_stride, gate_row};
+  KLLM_REQUIRE(!gate_sums || (gate_nsplit >= 1 && gate_width > 0 && gate_width <= vd && gate_row >= (long)H * gate_width),
+               "attn_generic: a gate of %d columns a head for values of %d, rows of %ld", gate_width, vd, gate_row);
   KLLM_REQUIRE(q && out && cache && positions && span_of_token && block_table,
                "attn_generic: null pointer");
   KLLM_REQUIRE(n > 0 && H > 0 && KV > 0 && H % KV == 0, "attn_generic: bad heads n=%d H=%d KV=%d", n,
@@ -143,11 +149,11 @@ extern "C" int kllm_attn_generic(const void* q, void* out, const void* cache, co
   if (dtype == DT_F32)
     hipLaunchKernelGGL(attn_generic_kernel<float>, grid, dim3(kAttnThreads), 0, stream,
                        (const float*)q, (float*)out, (const float*)cache, positions, span_of_token,
-                       block_table, max_pages, page_size, H, KV, hd, vd, window, chunk, sink, scale, slopes, keep_first);
+                       block_table, max_pages, page_size, H, KV, hd, vd, window, chunk, sinks, scale, slopes, keep_first, gate);
   else
     hipLaunchKernelGGL(attn_generic_kernel<bf16_t>, grid, dim3(kAttnThreads), 0, stream,
                        (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions,
-                       span_of_token, block_table, max_pages, page_size, H, KV, hd, vd, window, chunk, sink, scale, slopes, keep_first);
+                       span_of_token, block_table, max_pages, page_size, H, KV, hd, vd, window, chunk, sinks, scale, slopes, keep_first, gate);
   KLLM_CHECK_LAUNCH("attn_generic");
   return 0;
 }

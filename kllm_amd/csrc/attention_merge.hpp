@@ -16,7 +16,7 @@ namespace kllm {
 // round, for callers with few.)
 template <typename T, int DV, int R = 16>   // DV: elements of a head per lane (head size up to 64 DV); R: slices a round
 __device__ __forceinline__ void attn_merge_one(T* __restrict__ out, const float* __restrict__ part, int t, int h, int H,
-                                               int hd, int nslices, int lane) {
+                                               int hd, int nslices, int lane, const OutGate& gate) {
   const int stride = hd + 2;
   const float* p = part + ((long)t * H + h) * nslices * stride;
   float M = -INFINITY, denom = 0.f, o[DV];
@@ -54,7 +54,8 @@ __device__ __forceinline__ void attn_merge_one(T* __restrict__ out, const float*
   }
 #pragma unroll
   for (int v = 0; v < DV; ++v)
-    if (lane + 64 * v < hd) out[((long)t * H + h) * hd + lane + 64 * v] = from_f32<T>(o[v] / denom);
+    if (lane + 64 * v < hd)
+      out[((long)t * H + h) * hd + lane + 64 * v] = from_f32<T>(o[v] / denom * out_gate(gate, t, h, lane + 64 * v));
 }
 
 // The same for up to 64 slices and heads of up to 128 in one trip to memory instead of one per
@@ -63,7 +64,7 @@ __device__ __forceinline__ void attn_merge_one(T* __restrict__ out, const float*
 // weights go from lane to lane while the sums are added in the order of the slices.
 template <typename T, int DV, int R>   // R: 16, 32 or 64, at least the number of slices
 __device__ __forceinline__ void attn_merge_wide(T* __restrict__ out, const float* __restrict__ part, int t, int h, int H,
-                                                int hd, int nslices, int lane) {
+                                                int hd, int nslices, int lane, const OutGate& gate) {
   const int stride = hd + 2;
   const float* p = part + ((long)t * H + h) * nslices * stride;
   float os[DV][R];
@@ -93,35 +94,38 @@ __device__ __forceinline__ void attn_merge_wide(T* __restrict__ out, const float
   }
 #pragma unroll
   for (int v = 0; v < DV; ++v)
-    if (lane + 64 * v < hd) out[((long)t * H + h) * hd + lane + 64 * v] = from_f32<T>(o[v] / denom);
+    if (lane + 64 * v < hd)
+      out[((long)t * H + h) * hd + lane + 64 * v] = from_f32<T>(o[v] / denom * out_gate(gate, t, h, lane + 64 * v));
 }
 
 template <typename T, int DV, int R>
 __global__ __launch_bounds__(64) void attn_merge_wide_kernel(T* __restrict__ out, const float* __restrict__ part, int H,
-                                                             int hd, int nslices, const int* __restrict__ token_list) {
+                                                             int hd, int nslices, const int* __restrict__ token_list,
+                                                             const OutGate gate) {
   const int t = token_list ? token_list[blockIdx.x] : blockIdx.x;
-  attn_merge_wide<T, DV, R>(out, part, t, blockIdx.y, H, hd, nslices, threadIdx.x);
+  attn_merge_wide<T, DV, R>(out, part, t, blockIdx.y, H, hd, nslices, threadIdx.x, gate);
 }
 
 template <typename T, int DV>
 __global__ __launch_bounds__(64) void attn_merge_kernel(T* __restrict__ out,
                                                         const float* __restrict__ part, int H, int hd,
-                                                        int nslices, const int* __restrict__ token_list) {
+                                                        int nslices, const int* __restrict__ token_list,
+                                                        const OutGate gate) {
   const int t = token_list ? token_list[blockIdx.x] : blockIdx.x;
-  attn_merge_one<T, DV>(out, part, t, blockIdx.y, H, hd, nslices, threadIdx.x);
+  attn_merge_one<T, DV>(out, part, t, blockIdx.y, H, hd, nslices, threadIdx.x, gate);
 }
 
 // Launches the merge for `count` tokens (all, or those that token_list names).
 template <typename T>
 inline void launch_attn_merge(T* out, const float* part, int count, int H, int hd, int nslices,
-                              const int* token_list, hipStream_t stream) {
+                              const int* token_list, const OutGate& gate, hipStream_t stream) {
   const dim3 grid(count, H), block(64);
   if (nslices <= 64 && hd <= 128) {
     // (one trip to memory whatever the number of slices, and a lane asks for 2 + slices x DV
     // numbers instead of slices x (2 + DV); 64 slices of a head of 64: the merge 10 us -> 6,
     // 16 slices: a microsecond less)
 #define KLLM_MERGE_WIDE(DV, R) \
-    hipLaunchKernelGGL((attn_merge_wide_kernel<T, DV, R>), grid, block, 0, stream, out, part, H, hd, nslices, token_list)
+    hipLaunchKernelGGL((attn_merge_wide_kernel<T, DV, R>), grid, block, 0, stream, out, part, H, hd, nslices, token_list, gate)
     if (hd <= 64) {
       if (nslices <= 16) KLLM_MERGE_WIDE(1, 16); else if (nslices <= 32) KLLM_MERGE_WIDE(1, 32); else KLLM_MERGE_WIDE(1, 64);
     } else {
@@ -130,10 +134,10 @@ inline void launch_attn_merge(T* out, const float* part, int count, int H, int h
 #undef KLLM_MERGE_WIDE
     return;
   }
-  if (hd <= 64) hipLaunchKernelGGL((attn_merge_kernel<T, 1>), grid, block, 0, stream, out, part, H, hd, nslices, token_list);
-  else if (hd <= 128) hipLaunchKernelGGL((attn_merge_kernel<T, 2>), grid, block, 0, stream, out, part, H, hd, nslices, token_list);
-  else if (hd <= 192) hipLaunchKernelGGL((attn_merge_kernel<T, 3>), grid, block, 0, stream, out, part, H, hd, nslices, token_list);
-  else hipLaunchKernelGGL((attn_merge_kernel<T, 4>), grid, block, 0, stream, out, part, H, hd, nslices, token_list);
+  if (hd <= 64) hipLaunchKernelGGL((attn_merge_kernel<T, 1>), grid, block, 0, stream, out, part, H, hd, nslices, token_list, gate);
+  else if (hd <= 128) hipLaunchKernelGGL((attn_merge_kernel<T, 2>), grid, block, 0, stream, out, part, H, hd, nslices, token_list, gate);
+  else if (hd <= 192) hipLaunchKernelGGL((attn_merge_kernel<T, 3>), grid, block, 0, stream, out, part, H, hd, nslices, token_list, gate);
+  else hipLaunchKernelGGL((attn_merge_kernel<T, 4>), grid, block, 0, stream, out, part, H, hd, nslices, token_list, gate);
 }
 
 }  // namespace kllm

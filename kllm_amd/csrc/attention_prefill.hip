@@ -75,7 +75,8 @@ __global__ __launch_bounds__(64 * kPrefillWaves * PAR) __attribute__((amdgpu_wav
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ query_tiles, int n_tiles, const int* __restrict__ span_start,
     const int* __restrict__ span_pos, const int* __restrict__ block_table, int max_pages,
-    int page_size, unsigned page_magic, int H, int KV, int window, int chunk, int sink, int keep_first, float scale, const float* __restrict__ slopes, float* __restrict__ part) {
+    int page_size, unsigned page_magic, int H, int KV, int window, int chunk, const float* __restrict__ sinks, int keep_first,
+    float scale, const float* __restrict__ slopes, float* __restrict__ part, const OutGate gate) {
   typedef PrefillShape<HDT> S;
   constexpr int hd = S::hd, KS = S::KS, NB = S::NB, KT = S::KT, KLD = S::KLD, VLD = S::VLD, CPT = S::CPT;
   extern __shared__ __attribute__((aligned(16))) bf16_t tiles_lds[];   // [PAR][2][kBuf]
@@ -260,10 +261,11 @@ __global__ __launch_bounds__(64 * kPrefillWaves * PAR) __attribute__((amdgpu_wav
   const float grow_raw = kGrow / c2;                        // kGrow in units of raw scores
   float mc = 0.f;                                           // m * c2, 0 while m is -inf
   float m_limit = -INFINITY;                                // m + grow_raw
-  if (sink && par == 0 && slice == 0) {   // a key whose score is 0 and that has no value: where one group's maximum and sum start
-    m = 0.f;
+  if (sinks && par == 0 && slice == 0) {   // a key with a score of its own and no value: where one group's maximum and sum start
+    m = sinks[h] / scale;                     // in units of raw scores, as the maximum is
     l = 1.f;
-    m_limit = grow_raw;
+    mc = m * c2;
+    m_limit = m + grow_raw;
   }
   auto tile_math = [&](auto masked, int kb, const bf16_t* buf, bool kept_tile) {
     // ---- scores: this lane's key rows are kb + c and kb + 32 + c
@@ -463,9 +465,10 @@ __global__ __launch_bounds__(64 * kPrefillWaves * PAR) __attribute__((amdgpu_wav
   for (int r = 0; r < HDT; ++r)
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
+      const floatx4 og = out_gate4(gate, tq, h, 32 * r + 8 * b + 4 * g);
       bf16x4 v;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[j] = (bf16_t)(acc[r][4 * b + j] * inv);
+      for (int j = 0; j < 4; ++j) v[j] = (bf16_t)(acc[r][4 * b + j] * inv * og[j]);
       *reinterpret_cast<bf16x4*>(orow + 32 * r + 8 * b + 4 * g) = v;
     }
 }
@@ -477,13 +480,13 @@ constexpr int kMergeWaves = 8;   // (query, head) pairs of a workgroup of the me
 template <int DV>
 __global__ __launch_bounds__(64 * kMergeWaves) void attn_prefill_merge_kernel(
     bf16_t* __restrict__ out, const float* __restrict__ part, const int* __restrict__ query_tiles,
-    const int* __restrict__ span_start, int H, int hd, int nslices) {
+    const int* __restrict__ span_start, int H, int hd, int nslices, const OutGate gate) {
   const int tile = blockIdx.x / kQueryBlock;
   const int t = query_tiles[2 * tile] + blockIdx.x % kQueryBlock;
   if (t >= span_start[query_tiles[2 * tile + 1] + 1]) return;
   const int h = blockIdx.y * kMergeWaves + threadIdx.x / kWave;
   if (h >= H) return;
-  attn_merge_wide<bf16_t, DV, kPrefillMaxSlices>(out, part, t, h, H, hd, nslices, threadIdx.x % kWave);
+  attn_merge_wide<bf16_t, DV, kPrefillMaxSlices>(out, part, t, h, H, hd, nslices, threadIdx.x % kWave, gate);
 }
 
 // ---------------------------------------------------------------------------
@@ -502,7 +505,8 @@ __global__ __launch_bounds__(64 * kPrefillWaves) __attribute__((amdgpu_waves_per
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ query_tiles, int n_tiles, const int* __restrict__ span_start,
     const int* __restrict__ span_pos, const int* __restrict__ block_table, int max_pages,
-    int page_size, int H, int KV, int window, int chunk, int sink, float scale, const float* __restrict__ slopes) {
+    int page_size, int H, int KV, int window, int chunk, const float* __restrict__ sinks, float scale,
+    const float* __restrict__ slopes, const OutGate gate) {
   constexpr int hd = 32 * HDT;
   constexpr int KS = hd / 16;
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -613,10 +617,11 @@ __global__ __launch_bounds__(64 * kPrefillWaves) __attribute__((amdgpu_waves_per
   const float grow_raw = kGrow / c2;                        // kGrow in units of raw scores
   float mc = 0.f;                                           // m * c2, 0 while m is -inf
   float m_limit = -INFINITY;                                // m + grow_raw
-  if (sink && wave == 0) {                // a key whose score is 0 and that has no value: where one wave's maximum and sum start
-    m = 0.f;
+  if (sinks && wave == 0) {               // a key with a score of its own and no value: where one wave's maximum and sum start
+    m = sinks[h] / scale;
     l = 1.f;
-    m_limit = grow_raw;
+    mc = m * c2;
+    m_limit = m + grow_raw;
   }
   auto compute = [&](const Tile& cur, int kb) {
     // ---- scores: this lane's key row is kb + c
@@ -751,6 +756,7 @@ __global__ __launch_bounds__(64 * kPrefillWaves) __attribute__((amdgpu_waves_per
   for (int r = 0; r < HDT; ++r)
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
+      const floatx4 og = out_gate4(gate, tq, h, 32 * r + 8 * b + 4 * g);
       bf16x4 v;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
@@ -758,7 +764,7 @@ __global__ __launch_bounds__(64 * kPrefillWaves) __attribute__((amdgpu_waves_per
         float o = acc[r][i] * w0;
 #pragma unroll
         for (int w = 0; w < kPrefillWaves - 1; ++w) o += ww[w] * red[(w * kRows + 16 * r + i) * kWave + lane];
-        v[j] = (bf16_t)(o * inv);
+        v[j] = (bf16_t)(o * inv * og[j]);
       }
       *reinterpret_cast<bf16x4*>(orow + 32 * r + 8 * b + 4 * g) = v;
     }
@@ -768,7 +774,8 @@ template <int HDT, int PAR>
 static void launch_prefill_par(int grid, hipStream_t stream, const void* q, void* out, const void* cache,
                                const int* query_tiles, int n_tiles, const int* span_start,
                                const int* span_pos, const int* block_table, int max_pages, int page_size,
-                               int H, int KV, int window, int chunk, int sink, int keep_first, float scale, const float* slopes, float* part = nullptr, int nslices = 1) {
+                               int H, int KV, int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes,
+                               const OutGate& gate, float* part = nullptr, int nslices = 1) {
   typedef PrefillShape<HDT> S;
   const size_t lds = (size_t)PAR * 2 * S::kBuf * sizeof(bf16_t);   // also holds the groups' merge
   static int raised = 0;
@@ -780,11 +787,11 @@ static void launch_prefill_par(int grid, hipStream_t stream, const void* q, void
   const unsigned page_magic = (unsigned)(((1UL << 35) + page_size - 1) / page_size);   // ceil(2^35 / page_size)
   hipLaunchKernelGGL((attn_prefill_mfma_kernel<HDT, PAR>), dim3(grid, nslices), dim3(64 * kPrefillWaves * PAR), lds, stream,
                      (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, query_tiles, n_tiles,
-                     span_start, span_pos, block_table, max_pages, page_size, page_magic, H, KV, window, chunk, sink, keep_first, scale, slopes, part);
+                     span_start, span_pos, block_table, max_pages, page_size, page_magic, H, KV, window, chunk, sinks, keep_first, scale, slopes, part, gate);
   if (nslices > 1) {
     const dim3 mgrid(n_tiles * kQueryBlock, ceil_div(H, kMergeWaves));
     hipLaunchKernelGGL((attn_prefill_merge_kernel<(HDT + 1) / 2>), mgrid, dim3(64 * kMergeWaves), 0, stream,
-                       (bf16_t*)out, part, query_tiles, span_start, H, 32 * HDT, nslices);
+                       (bf16_t*)out, part, query_tiles, span_start, H, 32 * HDT, nslices, gate);
   }
 }
 
@@ -792,7 +799,7 @@ template <int HDT>
 static void launch_prefill_split(int n_tiles, hipStream_t stream, const void* q, void* out, const void* cache,
                                  const int* query_tiles, const int* span_start, const int* span_pos,
                                  const int* block_table, int max_pages, int page_size, int H, int KV,
-                                 int window, int chunk, int sink, float scale, const float* slopes) {
+                                 int window, int chunk, const float* sinks, float scale, const float* slopes, const OutGate& gate) {
   const size_t lds = (size_t)(kPrefillWaves - 1) * (HDT * 16 + 2) * kWave * sizeof(float);
   static int raised = 0;
   if (lds > 64 * 1024 && !raised) {
@@ -803,7 +810,7 @@ static void launch_prefill_split(int n_tiles, hipStream_t stream, const void* q,
   const int grid = n_tiles * (kQueryBlock / kQueryTile) * H;
   hipLaunchKernelGGL(attn_prefill_split_kernel<HDT>, dim3(grid), dim3(64 * kPrefillWaves), lds, stream,
                      (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, query_tiles, n_tiles,
-                     span_start, span_pos, block_table, max_pages, page_size, H, KV, window, chunk, sink, scale, slopes);
+                     span_start, span_pos, block_table, max_pages, page_size, H, KV, window, chunk, sinks, scale, slopes, gate);
 }
 
 // Which kernel.  One group of waves with the keys through LDS (three workgroups a CU) when
@@ -827,16 +834,16 @@ template <int HDT>
 static void launch_prefill(int grid, hipStream_t stream, const void* q, void* out, const void* cache,
                            const int* query_tiles, int n_tiles, const int* span_start,
                            const int* span_pos, const int* block_table, int max_pages, int page_size,
-                           int H, int KV, int window, int chunk, int sink, int keep_first, float scale, const float* slopes, long keys_total,
-                           int keys_longest, float* part, int nslices) {
+                           int H, int KV, int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes,
+                           long keys_total, int keys_longest, float* part, int nslices, const OutGate& gate) {
   const int cus = device_cus();
   // (the caller asked kllm_attn_prefill_slices: few blocks of a large head.  The slices' results
   // pass through memory and a second kernel, about 10 us for 512 queries of 32 heads; they pay
   // from about 1,280 keys to the longest block on, see there.)
   if (nslices > 1 && keys_longest >= kPrefillSliceFromKeys) {
     launch_prefill_par<HDT, PrefillShape<HDT>::kMaxPar>(grid, stream, q, out, cache, query_tiles, n_tiles, span_start,
-                                                        span_pos, block_table, max_pages, page_size, H, KV, window, chunk, sink,
-                                                        keep_first, scale, slopes, part, nslices);
+                                                        span_pos, block_table, max_pages, page_size, H, KV, window, chunk, sinks,
+                                                        keep_first, scale, slopes, gate, part, nslices);
     return;
   }
   bool chain_bound = true;
@@ -844,14 +851,14 @@ static void launch_prefill(int grid, hipStream_t stream, const void* q, void* ou
     chain_bound = 5 * (keys_total * H / cus) < 6 * (long)keys_longest;
   if (grid > 2 * cus || PrefillShape<HDT>::kMaxPar == 1 || (grid > cus && !chain_bound))
     launch_prefill_par<HDT, 1>(grid, stream, q, out, cache, query_tiles, n_tiles, span_start, span_pos,
-                               block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes);
+                               block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes, gate);
   else if (HDT >= 4 || 4 * grid > 3 * cus || keep_first > 0)   // (the kernel below reads one run of keys a query)
     launch_prefill_par<HDT, PrefillShape<HDT>::kMaxPar>(grid, stream, q, out, cache, query_tiles, n_tiles,
                                                         span_start, span_pos, block_table, max_pages, page_size,
-                                                        H, KV, window, chunk, sink, keep_first, scale, slopes);
+                                                        H, KV, window, chunk, sinks, keep_first, scale, slopes, gate);
   else
     launch_prefill_split<HDT>(n_tiles, stream, q, out, cache, query_tiles, span_start, span_pos, block_table,
-                              max_pages, page_size, H, KV, window, chunk, sink, scale, slopes);
+                              max_pages, page_size, H, KV, window, chunk, sinks, scale, slopes, gate);
 }
 
 }  // namespace kllm
@@ -877,8 +884,12 @@ extern "C" int kllm_attn_prefill_slices(int n_tiles, int H, int hd) {
 extern "C" int kllm_attn_prefill(const void* q, void* out, const void* cache, const int* query_tiles,
                                  int n_tiles, const int* span_start, const int* span_pos,
                                  const int* block_table, int max_pages, int page_size, int H, int KV,
-                                 int hd, int window, int chunk, int sink, int keep_first, float scale, const float* slopes, long keys_total, int keys_longest,
-                                 float* part, long part_floats, int nslices, int n_rows, int dtype, hipStream_t stream) {
+                                 int hd, int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes, long keys_total, int keys_longest,
+                                 float* part, long part_floats, int nslices, int n_rows, int dtype, const float* gate_sums, int gate_nsplit,
+                                 long gate_stride, long gate_row, int gate_width, hipStream_t stream) {
+  const OutGate gate = {gate_sums, gate_nsplit, gate_width, gate_stride, gate_row};
+  KLLM_REQUIRE(!gate_sums || (gate_nsplit >= 1 && gate_width > 0 && gate_width <= hd && gate_row >= (long)H * gate_width),
+               "attn_prefill: a gate of %d columns a head for heads of %d, rows of %ld", gate_width, hd, gate_row);
   KLLM_REQUIRE(q && out && cache && query_tiles && span_start && span_pos && block_table,
                "attn_prefill: null pointer");
   KLLM_REQUIRE(keys_total >= 0 && keys_longest >= 0, "attn_prefill: negative numbers of keys");
@@ -890,7 +901,7 @@ extern "C" int kllm_attn_prefill(const void* q, void* out, const void* cache, co
     KLLM_REQUIRE(keep_first == 0, "attn_prefill: the 32-bit kernels read one run of keys a query");
     KLLM_REQUIRE(max_pages > 0 && window >= 0 && chunk >= 0, "attn_prefill: bad table width, window or chunk");
     return attn_f32_prefill((const float*)q, (float*)out, (const float*)cache, query_tiles, n_tiles, span_start,
-                            span_pos, block_table, max_pages, page_size, H, KV, hd, window, chunk, sink, scale, slopes, stream);
+                            span_pos, block_table, max_pages, page_size, H, KV, hd, window, chunk, sinks, scale, slopes, gate, stream);
   }
   KLLM_REQUIRE(hd % 32 == 0 && hd >= 32 && hd <= 256 && (hd <= 128 || hd == 192 || hd == 256),
                "attn_prefill: head_dim %d is not built (32, 64, 96, 128, 192, 256)", hd);
@@ -912,8 +923,8 @@ extern "C" int kllm_attn_prefill(const void* q, void* out, const void* cache, co
 #define KLLM_PF(HDT)                                                                              \
   case HDT:                                                                                       \
     launch_prefill<HDT>(grid, stream, q, out, cache, query_tiles, n_tiles, span_start, span_pos,  \
-                        block_table, max_pages, page_size, H, KV, window, chunk, sink, keep_first, scale, slopes, keys_total, \
-                        keys_longest, part, nslices);                                             \
+                        block_table, max_pages, page_size, H, KV, window, chunk, sinks, keep_first, scale, slopes, keys_total, \
+                        keys_longest, part, nslices, gate);                                             \
     break
   switch (hd / 32) {
     KLLM_PF(1); KLLM_PF(2); KLLM_PF(3); KLLM_PF(4); KLLM_PF(6); KLLM_PF(8);

@@ -78,6 +78,37 @@ __host__ __device__ __forceinline__ int first_key(int pos, int window, int chunk
 
 __device__ __forceinline__ float sigmoid_f32(float v) { return 1.f / (1.f + expf(-v)); }
 
+// A gate on attention's output: the output's element d of head h is multiplied by the logistic
+// function of a sum of its own, taken where the output is written.  `sums` (null: no gate) points to
+// the gate's first column of float32 sums [nsplit][tokens][row]; a head has `width` columns, and
+// elements beyond them (padding, zero anyway) are not gated.
+struct OutGate {
+  const float* sums;
+  int nsplit, width;
+  long split_stride, row;
+};
+
+__device__ __forceinline__ float out_gate(const OutGate& g, long t, int h, int d) {
+  if (!g.sums || d >= g.width) return 1.f;
+  const float* at = g.sums + t * g.row + (long)h * g.width + d;
+  float z = 0.f;
+  for (int s = 0; s < g.nsplit; ++s) z += at[s * g.split_stride];
+  return sigmoid_f32(z);
+}
+
+// The same for elements d .. d + 3 (d a multiple of four), whose loads go out together.
+__device__ __forceinline__ floatx4 out_gate4(const OutGate& g, long t, int h, int d) {
+  if (!g.sums) return floatx4{1.f, 1.f, 1.f, 1.f};
+  const float* at = g.sums + t * g.row + (long)h * g.width;
+  floatx4 z = {0.f, 0.f, 0.f, 0.f};
+  for (int s = 0; s < g.nsplit; ++s)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) z[e] += at[s * g.split_stride + min(d + e, g.width - 1)];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) z[e] = sigmoid_f32(z[e]);
+  return z;
+}
+
 // A gate and the sum it gates, for kernels that take both: act(g) * u for the gates' activations,
 // or the clamped gate: with g' = min(g, limit) and u' = clamp(u, -limit, limit),
 // g' sigmoid(alpha g') (u' + 1).

@@ -67,6 +67,7 @@ static const Op kOps[] = {
     KLLM_CMD_OP(kllm_decayed_out),
     KLLM_CMD_OP(kllm_decayed_step),
     KLLM_CMD_OP(kllm_token_gate),
+    KLLM_CMD_OP(kllm_soft_cap),
 };
 constexpr int kNumOps = (int)(sizeof(kOps) / sizeof(kOps[0]));
 

@@ -212,13 +212,18 @@ int kllm_fused_linear(const void* x, int x_stride, const KllmLinearOut* out, con
  * head: slopes[h] * (query position - key position) is taken off the scaled score, a bias
  * that grows with the distance to the key.
  * `vd`: width of a value (a page holds keys [KV][slot][hd], then values [KV][vd][slot]);
- * `chunk` > 0: the query at position p reads no key before p - p % chunk; `sink` != 0: the
- * softmax's denominator has one more term, exp(0); `keep_first` > 0: the first keep_first
- * positions of a request stay readable behind the window (their pages are kept). */
+ * `chunk` > 0: the query at position p reads no key before p - p % chunk; `sinks` (null: none): the
+ * softmax's denominator of head h has one more term, exp(sinks[h]), neither scaled nor biased;
+ * `keep_first` > 0: the first keep_first positions of a request stay readable behind the window
+ * (their pages are kept).  A gate on the output (`gate_sums` null: none): element d of head h of
+ * token t is multiplied by the logistic function of the sum over gate_nsplit slices (gate_stride
+ * apart) of gate_sums[t * gate_row + h * gate_width + d]; elements from gate_width on are not gated. */
 int kllm_attn_generic(const void* q, void* out, const void* cache, const int* positions,
                       const int* span_of_token, const int* block_table, int max_pages,
                       int page_size, int n, int H, int KV, int hd, int vd, int window, int chunk,
-                      int sink, float scale, const float* slopes, int dtype, int keep_first, hipStream_t stream);
+                      const float* sinks, float scale, const float* slopes, int dtype, int keep_first,
+                      const float* gate_sums, int gate_nsplit, long gate_stride, long gate_row, int gate_width,
+                      hipStream_t stream);
 
 /* Decode attention on the matrix cores: every token's keys are cut into
  * `nslices` slices (1..256) that run side by side (bfloat16: a workgroup of 4
@@ -233,13 +238,14 @@ int kllm_attn_generic(const void* q, void* out, const void* cache, const int* po
 int kllm_attn_decode_slices(int n, int KV, int H, int hd, int dtype, int max_keys);
 /* Whether the float32 attention on the matrix cores takes this head size and page size. */
 int kllm_attn_f32_fits(int hd, int page_size);
-/* `chunk`, `sink` and `keep_first` in kllm_attn_decode and kllm_attn_prefill: as in kllm_attn_generic
+/* `chunk`, `sinks`, `keep_first` and the gate in kllm_attn_decode and kllm_attn_prefill: as in kllm_attn_generic
  * (kept first positions: bfloat16 only). */
 int kllm_attn_decode(const void* q, void* out, float* part, long part_floats, const void* cache,
                      const int* positions, const int* span_of_token, const int* block_table,
                      int max_pages, int page_size, int n, int H, int KV, int hd, int window,
-                     int chunk, int sink, int keep_first, float scale, const float* slopes, int nslices, int dtype,
-                     const int* token_list, int n_listed, hipStream_t stream);
+                     int chunk, const float* sinks, int keep_first, float scale, const float* slopes, int nslices, int dtype,
+                     const int* token_list, int n_listed, const float* gate_sums, int gate_nsplit, long gate_stride,
+                     long gate_row, int gate_width, hipStream_t stream);
 
 /* kllm_attn_decode without a workspace argument and without any allocation: for callers
  * that cannot allocate device memory (code under HIP graph capture, tight serving loops,
@@ -271,8 +277,9 @@ int kllm_attn_decode_static(const void* q, void* out, const void* cache, const i
 int kllm_attn_prefill(const void* q, void* out, const void* cache, const int* query_tiles,
                       int n_tiles, const int* span_start, const int* span_pos,
                       const int* block_table, int max_pages, int page_size, int H, int KV, int hd,
-                      int window, int chunk, int sink, int keep_first, float scale, const float* slopes, long keys_total,
+                      int window, int chunk, const float* sinks, int keep_first, float scale, const float* slopes, long keys_total,
                       int keys_longest, float* part, long part_floats, int nslices, int n_rows, int dtype,
+                      const float* gate_sums, int gate_nsplit, long gate_stride, long gate_row, int gate_width,
                       hipStream_t stream);
 /* nslices of kllm_attn_prefill: how many workgroups share out the keys of a block and head
  * (1: none; more where few blocks of a large head would leave CUs idle; taken only when
@@ -298,12 +305,16 @@ int kllm_unary_act(const float* in, int nsplit, long split_stride, int in_row_st
 /* The norm of a layer whose sub-layers run side by side.  v = x[src] + mult * (sum of d1's ns1
  * slices + sum of d2's ns2 slices + bias) (each of d1, d2, bias may be null); x[src] = v when
  * write_x; when out is not null, out[r] = v / sqrt(mean over the channel's group of v^2 + eps)
- * * w, the d channels being cut into `groups` equal consecutive groups (1: an RMS norm).
+ * * w, the d channels being cut into `groups` equal consecutive groups (1: an RMS norm).  With
+ * `norm_bias` [d] (one group) the norm is taken around the row's mean: out[r] = (v - mean) /
+ * sqrt(mean of (v - mean)^2 + eps) * w + norm_bias.
  * src = rows[r] when rows is given (then write_x must be 0), else r. */
 int kllm_group_norm_add(float* x, const float* d1, int ns1, long st1, const float* d2, int ns2, long st2,
                         const float* bias, float mult, const float* w, void* out, int out_dtype,
                         const int* rows, int n, int d, int groups, float eps, int write_x,
-                        hipStream_t stream);
+                        const float* norm_bias, hipStream_t stream);
+/* x[i] = cap * tanh(x[i] / cap), count numbers in place. */
+int kllm_soft_cap(float* x, long count, float cap, hipStream_t stream);
 
 /* Between the query/key product and attention where queries and keys are normalised over the
  * whole projection.  qk holds the sums [nsplit][n][(H + KV) * hd + KV * dv] (queries, keys,
@@ -494,14 +505,16 @@ int kllm_normed_sum(float* out, const float* a, int na, long stride_a, float sa,
  * first `rot` elements of every query and key head, writes q_out [n][H][width] and the pages (keys
  * [KV][slot][width], values [KV][width][slot], times v_scale; zeros beyond the heads' own width).
  * `single`: every span is one token; the state's field then takes the new inputs in the same launch
- * (otherwise kllm_conv_state_update follows). */
+ * (otherwise kllm_conv_state_update follows).  Without weights (conv_w null, taps 1) nothing is
+ * convolved, and `bias` [channels] (null: none) is added; without a cache (null, KV 0) there are
+ * queries only. */
 int kllm_qkv_conv_append(const float* sums, int nsplit, long split_stride, int row_len, int col0,
                          const float* conv_w, int taps, float* state, long slot_stride, int single,
                          const float* cos_t, const float* sin_t, int rot, int interleaved, float v_scale, void* q_out,
                          void* cache, const int* positions, const int* span_of_token, const int* slots,
                          const int* span_start, const int* span_pos, const int* block_table, int max_pages,
                          int page_size, int n, int H, int KV, int dk, int dv, int width, int dtype,
-                         hipStream_t stream);
+                         const float* bias, hipStream_t stream);
 
 /* ---- linear attention with decays (decayed.hip) ----
  * `sums` are float32 sums [nsplit][n][row] of a step's projections, *_col the first column of a
@@ -562,11 +575,15 @@ int kllm_latent_norm(const float* in, int nsplit, long split_stride, long in_str
 int kllm_latent_query(const float* q, int nsplit, long split_stride, const void* w_uk, const float* cos_t,
                       const float* sin_t, void* out, int n, int H, int d, int dr, int rank, int dtype,
                       int transposed, hipStream_t stream);
+/* window > 0: the query at position p reads the keys (p - window, p] (pages behind them may be gone). */
 int kllm_attn_latent(const void* q, void* out, const void* cache, const int* positions, const int* span_of_token,
                      const int* block_table, int max_pages, int page_size, int n, int H, int row, int rank,
-                     float scale, int dtype, int mode, float* part, long part_floats, int nslices, hipStream_t stream);
+                     float scale, int dtype, int mode, float* part, long part_floats, int nslices, int window,
+                     hipStream_t stream);
+/* gate: sums with one column an element, or (gate_by_head) one a head, or null. */
 int kllm_latent_out(const void* attended, const void* w_uv, const float* gate, int nsplit, long split_stride,
-                    long gate_stride, void* out, int n, int H, int dv, int rank, int dtype, hipStream_t stream);
+                    long gate_stride, void* out, int n, int H, int dv, int rank, int dtype, int gate_by_head,
+                    hipStream_t stream);
 
 #ifdef __cplusplus
 }

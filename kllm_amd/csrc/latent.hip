@@ -8,8 +8,10 @@
 //                      last dr (halves paired), appended to the pages (one row of rank + dr a slot)
 //   latent_query       sums of W_uq c_q -> per head [W_uk,h^T q_h | rotated q_h], rank + dr wide
 //   attn_latent        one workgroup a (token, head): online softmax over 256 keys at a time,
-//                      the values being the first rank elements of the cached rows
+//                      the values being the first rank elements of the cached rows; with a window
+//                      the last `window` keys only (pages behind it may be gone)
 //   latent_out         per head W_uv,h times the attended latent, times sigmoid of the gate's sums
+//                      (one gate an element, or one a head)
 //
 // Scores, softmax, norms and rotation are 32-bit; the cached rows, the folded queries and the
 // attended latents are stored in the compute type.
@@ -141,13 +143,14 @@ template <typename T>
 __global__ __launch_bounds__(kLatThreads) void attn_latent_kernel(
     const T* __restrict__ q, T* __restrict__ out, const T* __restrict__ cache, const int* __restrict__ positions,
     const int* __restrict__ span_of_token, const int* __restrict__ block_table, int max_pages, int page_size, int H,
-    int row, int rank, float scale) {
+    int row, int rank, float scale, int window) {
   __shared__ float qs[kLatMaxRow];
   __shared__ float ps[kLatThreads];
   __shared__ float red[16];
   const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const long page_elems = (long)page_size * (row + rank);
   const int len = positions[t] + 1;
+  const int lo = first_key(len - 1, window, 0);
   const int* table = block_table + (long)span_of_token[t] * max_pages;
   const T* qrow = q + ((long)t * H + h) * row;
   for (int i = tid; i < row; i += kLatThreads) qs[i] = to_f32(qrow[i]);
@@ -156,7 +159,7 @@ __global__ __launch_bounds__(kLatThreads) void attn_latent_kernel(
   float acc[kLatMaxPer];
 #pragma unroll
   for (int c = 0; c < kLatMaxPer; ++c) acc[c] = 0.f;
-  for (int base = 0; base < len; base += kLatThreads) {
+  for (int base = lo; base < len; base += kLatThreads) {
     const int key = base + tid;
     float s = -INFINITY;
     if (key < len) {
@@ -217,7 +220,8 @@ template <int NR, int KS>
 __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ span_of_token, const int* __restrict__ block_table,
-    int max_pages, int page_size, unsigned page_magic, int H, int row, int rank, float scale, float* __restrict__ part) {
+    int max_pages, int page_size, unsigned page_magic, int H, int row, int rank, float scale, int window,
+    float* __restrict__ part) {
   extern __shared__ float lat_red[];            // [kLatWaves - 1][NR * 4 + 2][64]
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   const int g = lane / 16, c = lane % 16;
@@ -225,6 +229,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
   const int head = min(h0 + c, H - 1);
   const bool head_ok = h0 + c < H;
   const int len = positions[t] + 1;
+  const int lo = first_key(len - 1, window, 0);        // the first key that is read
   const int* table = block_table + (long)span_of_token[t] * max_pages;
   const long page_elems = (long)page_size * (row + rank);
   const int ksteps = (row + 31) / 32, nr = rank / 16;
@@ -246,7 +251,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
   // tokens and heads alone leave CUs idle) and, within a slice, to the waves.
   const int nslices = gridDim.z, slice = blockIdx.z;
   const int tiles = (len + 31) / 32;
-  for (int tile = slice * kLatWaves + wave; tile < tiles; tile += kLatWaves * nslices) {
+  for (int tile = lo / 32 + slice * kLatWaves + wave; tile < tiles; tile += kLatWaves * nslices) {
     const int kb = tile * 32;
     // a half (16 keys) lies in one page (pages hold a multiple of 16 slots)
     const bf16_t* pbase[2];
@@ -255,9 +260,9 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       const int k0 = kb + 16 * u;
-      live[u] = k0 < len;
+      live[u] = k0 < len && k0 + 16 > lo;                    // (a half behind the window may lie in a page that is gone)
       const int pi = live[u] ? (int)(__umulhi((unsigned)k0, page_magic) >> 3) : 0;   // k0 / page_size (see the launch)
-      const int page = table[pi];
+      const int page = live[u] ? table[pi] : 0;
       pbase[u] = cache + (long)page * page_elems;
       slot0[u] = live[u] ? k0 - pi * page_size : 0;
     }
@@ -288,7 +293,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int key = kb + 16 * u + 4 * g + i;
-        s[u][i] = key < len ? s[u][i] * scale : -INFINITY;
+        s[u][i] = (key < len && key >= lo) ? s[u][i] * scale : -INFINITY;
         tmax = fmaxf(tmax, s[u][i]);
       }
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
@@ -406,7 +411,7 @@ template <int NR, int KS>
 __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ span_of_token, const int* __restrict__ block_table,
-    int max_pages, int page_size, unsigned page_magic, int n, int H, int row, int rank, float scale) {
+    int max_pages, int page_size, unsigned page_magic, int n, int H, int row, int rank, float scale, int window) {
   extern __shared__ __attribute__((aligned(16))) bf16_t lat_tiles[];
   // page of a key without a division: page_magic = ceil(2^35 / page_size) from the host, exact for
   // keys below 2^24 and pages of up to 2,048 slots (checked at the launch)
@@ -424,6 +429,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
   const bool head_ok = h0 + c < H;
   const int my_span = span_of_token[t];
   const int len = positions[t] + 1;
+  const int lo = first_key(len - 1, window, 0);
   const long page_elems = (long)page_size * (row + rank);
   const int ksteps = (row + 31) / 32, nr = rank / 16;
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -446,6 +452,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
     int last = first;
     while (last + 1 < rows_here && span_of_token[t_first + last + 1] == span) ++last;
     const int group_len = positions[t_first + last] + 1;      // the group's last token reads the most keys
+    const int group_lo = first_key(positions[t_first + first], window, 0);   // ... and its first the earliest (pages before it may be gone)
     const bool mine = token_ok && wave >= first && wave <= last;
     const int* table = block_table + (long)span * max_pages;
     // ---- a tile's way into LDS: 16-byte pieces (a half, 16 keys, lies in one page).  For the built
@@ -459,14 +466,14 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
     auto k_piece = [&](int i, int kb) -> bf16x8 {
       const int kr = i / row8;                                // (for the built sizes: unrolled, i and row8 known per thread before the loop)
       const int key = kb + kr;
-      if (i >= 32 * row8 || key >= group_len) return zero8;
+      if (i >= 32 * row8 || key >= group_len || key < group_lo) return zero8;
       const int pi = page_index(key);
       const long pg = table[pi];
       return *reinterpret_cast<const bf16x8*>(cache + pg * page_elems + (long)(key - pi * page_size) * row + 8 * (i - kr * row8));
     };
     auto v_piece = [&](int i, int kb) -> bf16x8 {             // 8 keys of one element
       const int e = i / 4, key = kb + 8 * (i % 4);
-      if (e >= rank || key >= group_len) return zero8;
+      if (e >= rank || key >= group_len || key + 8 <= group_lo) return zero8;
       const int pi = page_index(key);
       const long pg = table[pi];
       bf16x8 v = *reinterpret_cast<const bf16x8*>(cache + pg * page_elems + (long)page_size * row + (long)e * page_size +
@@ -496,8 +503,9 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
       return T;
     };
     Stage st;
-    if constexpr (KS > 0) st = fetch(0);
-    for (int kb = 0; kb < group_len; kb += 32) {
+    const int kb0 = group_lo / 32 * 32;
+    if constexpr (KS > 0) st = fetch(kb0);
+    for (int kb = kb0; kb < group_len; kb += 32) {
       __syncthreads();                                        // the tile before this one has been read
       if constexpr (KS > 0) {
 #pragma unroll
@@ -512,7 +520,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
       if constexpr (KS > 0) {
         if (kb + 32 < group_len) st = fetch(kb + 32);         // (the same for all: no barrier inside)
       }
-      if (!mine || kb >= len) continue;
+      if (!mine || kb >= len || kb + 32 <= lo) continue;
       // ---- scores
       floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
       auto score_step = [&](int kk, const bf16x8& qb) {
@@ -539,12 +547,12 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int key = kb + 16 * u + 4 * g + i;
-          s[u][i] = key < len ? s[u][i] * scale : -INFINITY;
+          s[u][i] = (key < len && key >= lo) ? s[u][i] * scale : -INFINITY;
           tmax = fmaxf(tmax, s[u][i]);
         }
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
       tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
-      const float m_new = fmaxf(m, tmax);                    // finite: kb < len
+      const float m_new = fmaxf(m, tmax);                    // finite: the tile holds a key of this token
       const float alpha = expf(m - m_new);
       bf16x8 pb;
       float psum = 0.f;
@@ -617,7 +625,7 @@ __global__ __launch_bounds__(kLatThreads) void attn_latent_merge_kernel(const fl
 template <int NR, int KS>
 static void launch_latent_mfma(const void* q, void* out, const void* cache, const int* positions, const int* span_of_token,
                                const int* block_table, int max_pages, int page_size, int n, int H, int row, int rank,
-                               float scale, float* part, int nslices, hipStream_t stream) {
+                               float scale, int window, float* part, int nslices, hipStream_t stream) {
   const size_t lds = (size_t)(kLatWaves - 1) * (NR * 4 + 2) * kWave * sizeof(float);
   const unsigned page_magic = (unsigned)(((1ull << 35) + page_size - 1) / page_size);
   static int raised = 0;
@@ -634,21 +642,21 @@ static void launch_latent_mfma(const void* q, void* out, const void* cache, cons
     }
     hipLaunchKernelGGL((attn_latent_block_kernel<NR, KS>), dim3((n + kLatWaves - 1) / kLatWaves, (H + 15) / 16), dim3(64 * kLatWaves),
                        tiles, stream, (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, span_of_token,
-                       block_table, max_pages, page_size, page_magic, n, H, row, rank, scale);
+                       block_table, max_pages, page_size, page_magic, n, H, row, rank, scale, window);
     return;
   }
   hipLaunchKernelGGL((attn_latent_mfma_kernel<NR, KS>), dim3(n, (H + 15) / 16, nslices), dim3(64 * kLatWaves), lds, stream,
                      (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, span_of_token, block_table, max_pages,
-                     page_size, page_magic, H, row, rank, scale, part);
+                     page_size, page_magic, H, row, rank, scale, window, part);
   if (nslices > 1)
     hipLaunchKernelGGL(attn_latent_merge_kernel, dim3(n * H), dim3(kLatThreads), 0, stream, part, (bf16_t*)out, rank, nslices);
 }
 
-// attended: [n][H][rank]; w_uv [H * dv][rank]; gate: [nsplit][n][H * dv] sums or null.
+// attended: [n][H][rank]; w_uv [H * dv][rank]; gate: [nsplit][n][H * dv] sums ([H] with by_head) or null.
 template <typename T>
 __global__ __launch_bounds__(kLatThreads) void latent_out_kernel(
     const T* __restrict__ attended, const T* __restrict__ w_uv, const float* __restrict__ gate, int nsplit,
-    long split_stride, long gate_stride, T* __restrict__ out, int H, int dv, int rank) {
+    long split_stride, long gate_stride, int by_head, T* __restrict__ out, int H, int dv, int rank) {
   extern __shared__ float al[];          // [rank]
   const long t = blockIdx.x;
   const int h = blockIdx.y, tid = threadIdx.x;
@@ -662,7 +670,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_out_kernel(
     const long col = (long)h * dv + j;
     if (gate) {
       float g = 0.f;
-      for (int s = 0; s < nsplit; ++s) g += gate[s * split_stride + t * gate_stride + col];
+      for (int s = 0; s < nsplit; ++s) g += gate[s * split_stride + t * gate_stride + (by_head ? h : col)];
       acc *= sigmoid_f32(g);
     }
     out[t * H * dv + col] = from_f32<T>(acc);
@@ -677,7 +685,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_out_kernel(
 //                 transposed once, when the weights are bound), and the rotated part beside it
 __global__ __launch_bounds__(kLatThreads) void latent_out_mfma_kernel(
     const bf16_t* __restrict__ attended, const bf16_t* __restrict__ w_uv, const float* __restrict__ gate, int nsplit,
-    long split_stride, long gate_stride, bf16_t* __restrict__ out, int n, int H, int dv, int rank) {
+    long split_stride, long gate_stride, int by_head, bf16_t* __restrict__ out, int n, int H, int dv, int rank) {
   const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   const int g = lane / 16, c = lane % 16;
   const int h = blockIdx.y;
@@ -703,7 +711,7 @@ __global__ __launch_bounds__(kLatThreads) void latent_out_mfma_kernel(
     float v = acc[i];
     if (gate) {
       float gs = 0.f;
-      for (int s = 0; s < nsplit; ++s) gs += gate[s * split_stride + tt * gate_stride + col];
+      for (int s = 0; s < nsplit; ++s) gs += gate[s * split_stride + tt * gate_stride + (by_head ? h : col)];
       v *= sigmoid_f32(gs);
     }
     out[(long)tt * H * dv + col] = (bf16_t)v;
@@ -832,11 +840,11 @@ extern "C" int kllm_latent_query(const float* q, int nsplit, long split_stride, 
 extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, const int* positions,
                                 const int* span_of_token, const int* block_table, int max_pages, int page_size, int n,
                                 int H, int row, int rank, float scale, int dtype, int mode, float* part, long part_floats, int nslices,
-                                hipStream_t stream) {
+                                int window, hipStream_t stream) {
   KLLM_REQUIRE(q && out && cache && positions && span_of_token && block_table, "attn_latent: null pointer");
   KLLM_REQUIRE(n > 0 && H > 0 && H <= 65535 && rank > 0 && rank <= row && row <= kLatMaxRow,
                "attn_latent: bad sizes n=%d H=%d row=%d rank=%d (rows of up to %d)", n, H, row, rank, kLatMaxRow);
-  KLLM_REQUIRE(max_pages > 0 && page_size > 0, "attn_latent: bad cache sizes");
+  KLLM_REQUIRE(max_pages > 0 && page_size > 0 && window >= 0, "attn_latent: bad cache sizes or window");
   KLLM_REQUIRE(dtype == DT_F32 || dtype == DT_BF16, "attn_latent: unknown dtype %d", dtype);
   if (dtype == DT_BF16 && mode != 1 && rank % 16 == 0 && row % 8 == 0 && rank <= 512 && page_size % 16 == 0 &&
       page_size <= 2048 && (long)max_pages * page_size <= (1L << 24) &&
@@ -846,7 +854,7 @@ extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, con
                  nslices, rank);
     // the latent's accumulators and the query's pieces in registers: built for ranks up to 128, 256 and
     // 512 with rows of up to 256, 384 and 640; longer rows ask for the query at every tile
-#define KLLM_LAT(NR, KS) launch_latent_mfma<NR, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, H, row, rank, scale, part, nslices, stream)
+#define KLLM_LAT(NR, KS) launch_latent_mfma<NR, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, H, row, rank, scale, window, part, nslices, stream)
     if (rank <= 128) { if (row <= 256) KLLM_LAT(8, 8); else KLLM_LAT(8, 0); }
     else if (rank <= 256) { if (row <= 384) KLLM_LAT(16, 12); else KLLM_LAT(16, 0); }
     else { if (row <= 640) KLLM_LAT(32, 20); else KLLM_LAT(32, 0); }
@@ -857,17 +865,17 @@ extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, con
   if (dtype == DT_F32)
     hipLaunchKernelGGL(attn_latent_kernel<float>, dim3(n, H), dim3(kLatThreads), 0, stream, (const float*)q,
                        (float*)out, (const float*)cache, positions, span_of_token, block_table, max_pages, page_size, H,
-                       row, rank, scale);
+                       row, rank, scale, window);
   else
     hipLaunchKernelGGL(attn_latent_kernel<bf16_t>, dim3(n, H), dim3(kLatThreads), 0, stream, (const bf16_t*)q,
                        (bf16_t*)out, (const bf16_t*)cache, positions, span_of_token, block_table, max_pages, page_size,
-                       H, row, rank, scale);
+                       H, row, rank, scale, window);
   KLLM_CHECK_LAUNCH("attn_latent");
   return 0;
 }
 
 extern "C" int kllm_latent_out(const void* attended, const void* w_uv, const float* gate, int nsplit, long split_stride,
-                               long gate_stride, void* out, int n, int H, int dv, int rank, int dtype,
+                               long gate_stride, void* out, int n, int H, int dv, int rank, int dtype, int gate_by_head,
                                hipStream_t stream) {
   KLLM_REQUIRE(attended && w_uv && out, "latent_out: null pointer");
   KLLM_REQUIRE(n > 0 && H > 0 && H <= 65535 && dv > 0 && rank > 0 && rank <= 8192 && (!gate || nsplit >= 1),
@@ -875,18 +883,18 @@ extern "C" int kllm_latent_out(const void* attended, const void* w_uv, const flo
   KLLM_REQUIRE(dtype == DT_F32 || dtype == DT_BF16, "latent_out: unknown dtype %d", dtype);
   if (dtype == DT_BF16 && rank % 32 == 0 && ((uintptr_t)attended & 15) == 0 && ((uintptr_t)w_uv & 15) == 0) {
     hipLaunchKernelGGL(latent_out_mfma_kernel, dim3((n + 15) / 16, H, (dv + 63) / 64), dim3(kLatThreads), 0, stream,
-                       (const bf16_t*)attended, (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride, (bf16_t*)out,
-                       n, H, dv, rank);
+                       (const bf16_t*)attended, (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride, gate_by_head,
+                       (bf16_t*)out, n, H, dv, rank);
     KLLM_CHECK_LAUNCH("latent_out");
     return 0;
   }
   const size_t lds = (size_t)rank * sizeof(float);
   if (dtype == DT_F32)
     hipLaunchKernelGGL(latent_out_kernel<float>, dim3(n, H), dim3(kLatThreads), lds, stream, (const float*)attended,
-                       (const float*)w_uv, gate, nsplit, split_stride, gate_stride, (float*)out, H, dv, rank);
+                       (const float*)w_uv, gate, nsplit, split_stride, gate_stride, gate_by_head, (float*)out, H, dv, rank);
   else
     hipLaunchKernelGGL(latent_out_kernel<bf16_t>, dim3(n, H), dim3(kLatThreads), lds, stream, (const bf16_t*)attended,
-                       (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride, (bf16_t*)out, H, dv, rank);
+                       (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride, gate_by_head, (bf16_t*)out, H, dv, rank);
   KLLM_CHECK_LAUNCH("latent_out");
   return 0;
 }

@@ -1,7 +1,8 @@
 // Per-token steps around the products of layers that are not Llama's: additive sinusoidal
 // positions, a gate that a vector looked up by the token multiplies, an activation without a gate (with learned constants), and the norm of a layer
 // whose sub-layers run side by side: it adds a scaled sum of up to two sub-layers' outputs
-// and a bias to the residual stream and normalises the result in groups of channels.
+// and a bias to the residual stream and normalises the result in groups of channels, or around
+// its mean; and a soft cap on the logits.
 // Everything here is computed in 32-bit.
 #include <math.h>
 
@@ -68,11 +69,13 @@ constexpr int kGroupNormThreads = 256;
 // x[src] = v when write_x; out[r] = v / sqrt(mean over the channel's group of v^2 + eps) * w.
 // A group's sum of squares is taken by one wave over a fixed cut of the group, in a fixed
 // order, so a row's result does not depend on what else the launch holds.
-template <typename TOUT>
+// CENTRED (one group): the row's mean is taken off first, the squares are those of the
+// deviations, and `wb` is added: (v - mean) / sqrt(mean of (v - mean)^2 + eps) * w + wb.
+template <typename TOUT, bool CENTRED>
 __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_kernel(
     float* __restrict__ x, const float* __restrict__ d1, int ns1, long st1, const float* __restrict__ d2, int ns2,
-    long st2, const float* __restrict__ bias, float mult, const float* __restrict__ w, TOUT* __restrict__ out,
-    const int* __restrict__ rows, int d, int groups, int segs, float eps, int write_x) {
+    long st2, const float* __restrict__ bias, float mult, const float* __restrict__ w, const float* __restrict__ wb,
+    TOUT* __restrict__ out, const int* __restrict__ rows, int d, int groups, int segs, float eps, int write_x) {
   extern __shared__ float v_lds[];          // [d] the row, then [groups * segs] partial sums
   float* part = v_lds + d;
   const long r = blockIdx.x;
@@ -96,6 +99,14 @@ __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_kernel(
   }
   if (!out) return;
   __syncthreads();
+  if constexpr (CENTRED) {
+    __shared__ float red[16];
+    float sum = 0.f;
+    for (int i = tid; i < d; i += kGroupNormThreads) sum += v_lds[i];
+    const float mean = block_sum(sum, red) / (float)d;
+    for (int i = tid; i < d; i += kGroupNormThreads) v_lds[i] -= mean;
+    __syncthreads();
+  }
   const int lane = tid % kWave, wave = tid / kWave, nwaves = kGroupNormThreads / kWave;
   const int gsz = d / groups;
   const int seg_len = (gsz + segs - 1) / segs;
@@ -113,7 +124,8 @@ __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_kernel(
     float ss = 0.f;
     for (int sg = 0; sg < segs; ++sg) ss += part[g * segs + sg];
     const float rstd = 1.f / sqrtf(ss / (float)gsz + eps);
-    out[r * d + i] = from_f32<TOUT>(v_lds[i] * rstd * w[i]);
+    const float y = v_lds[i] * rstd * w[i];
+    out[r * d + i] = from_f32<TOUT>(CENTRED ? y + wb[i] : y);
   }
 }
 
@@ -121,11 +133,11 @@ __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_kernel(
 // channels: a thread keeps its channels in registers, four at a time, and every load is 16 bytes.
 constexpr int kGroupNormMaxGroups = 8;
 
-template <typename TOUT, int KEEP>
+template <typename TOUT, int KEEP, bool CENTRED>
 __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_vec_kernel(
     float* __restrict__ x, const float* __restrict__ d1, int ns1, long st1, const float* __restrict__ d2, int ns2,
-    long st2, const float* __restrict__ bias, float mult, const float* __restrict__ w, TOUT* __restrict__ out,
-    const int* __restrict__ rows, int d, int groups, float eps, int write_x) {
+    long st2, const float* __restrict__ bias, float mult, const float* __restrict__ w, const float* __restrict__ wb,
+    TOUT* __restrict__ out, const int* __restrict__ rows, int d, int groups, float eps, int write_x) {
   __shared__ float red[16];
   __shared__ float rstd_g[kGroupNormMaxGroups];
   const long r = blockIdx.x;
@@ -156,6 +168,18 @@ __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_vec_kernel(
     }
   }
   if (!out) return;
+  if constexpr (CENTRED) {
+    float sum = 0.f;
+#pragma unroll
+    for (int it = 0; it < KEEP; ++it)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) sum += v[it][e];                     // (zeros beyond the row)
+    const float mean = block_sum(sum, red) / (float)d;
+#pragma unroll
+    for (int it = 0; it < KEEP; ++it)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[it][e] -= mean;                    // (beyond the row: not looked at below)
+  }
   const int gsz = d / groups;
   for (int g = 0; g < groups; ++g) {
     float ss = 0.f;
@@ -178,16 +202,29 @@ __global__ __launch_bounds__(kGroupNormThreads) void group_norm_add_vec_kernel(
     const floatx4 wv = *reinterpret_cast<const floatx4*>(w + 4 * c);
     TOUT o[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o[e] = from_f32<TOUT>(v[it][e] * rstd * wv[e]);
+    for (int e = 0; e < 4; ++e) o[e] = from_f32<TOUT>(CENTRED ? fmaf(v[it][e] * rstd, wv[e], wb[4 * c + e]) : v[it][e] * rstd * wv[e]);
     TOUT* dst = out + r * d + 4 * c;
 #pragma unroll
     for (int e = 0; e < 4; ++e) dst[e] = o[e];
   }
 }
 
+// x = cap * tanh(x / cap)
+__global__ void soft_cap_kernel(float* __restrict__ x, long count, float cap, float inv_cap) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < count) x[i] = cap * tanhf(x[i] * inv_cap);
+}
+
 }  // namespace kllm
 
 using namespace kllm;
+
+extern "C" int kllm_soft_cap(float* x, long count, float cap, hipStream_t stream) {
+  KLLM_REQUIRE(x && count > 0 && cap > 0.f, "soft_cap: %ld numbers, cap %g", count, cap);
+  hipLaunchKernelGGL(soft_cap_kernel, dim3(ceil_div(count, 256)), dim3(256), 0, stream, x, count, cap, 1.f / cap);
+  KLLM_CHECK_LAUNCH("soft_cap");
+  return 0;
+}
 
 extern "C" int kllm_add_sinusoid(float* x, const int* positions, int n, int d, double base, hipStream_t stream) {
   KLLM_REQUIRE(x && positions, "add_sinusoid: null pointer");
@@ -243,7 +280,8 @@ extern "C" int kllm_token_gate(const float* sums, int nsplit, long split_stride,
 extern "C" int kllm_group_norm_add(float* x, const float* d1, int ns1, long st1, const float* d2, int ns2, long st2,
                                    const float* bias, float mult, const float* w, void* out, int out_dtype,
                                    const int* rows, int n, int d, int groups, float eps, int write_x,
-                                   hipStream_t stream) {
+                                   const float* norm_bias, hipStream_t stream) {
+  KLLM_REQUIRE(!norm_bias || groups == 1, "group_norm_add: a norm around the mean takes the row in one group, not %d", groups);
   KLLM_REQUIRE(x, "group_norm_add: null pointer");
   KLLM_REQUIRE(n > 0 && d > 0 && groups > 0 && d % groups == 0, "group_norm_add: %d channels in %d groups (n=%d)", d,
                groups, n);
@@ -253,18 +291,23 @@ extern "C" int kllm_group_norm_add(float* x, const float* d1, int ns1, long st1,
   KLLM_REQUIRE(out_dtype == DT_F32 || out_dtype == DT_BF16, "group_norm_add: unknown dtype %d", out_dtype);
   const bool aligned = ((uintptr_t)x & 15) == 0 && (!d1 || (((uintptr_t)d1 & 15) == 0 && st1 % 4 == 0)) &&
                        (!d2 || (((uintptr_t)d2 & 15) == 0 && st2 % 4 == 0)) && (!bias || ((uintptr_t)bias & 15) == 0) &&
-                       (!w || ((uintptr_t)w & 15) == 0);
+                       (!w || ((uintptr_t)w & 15) == 0) && (!norm_bias || ((uintptr_t)norm_bias & 15) == 0);
   if (aligned && d % 4 == 0 && (d / groups) % 4 == 0 && groups <= kGroupNormMaxGroups && d <= 4 * kGroupNormThreads * 8) {
     const int keep = ceil_div(d / 4, kGroupNormThreads);
-#define KLLM_GN(T, KEEP)                                                                                          \
-  hipLaunchKernelGGL((group_norm_add_vec_kernel<T, KEEP>), dim3(n), dim3(kGroupNormThreads), 0, stream, x, d1, ns1, \
-                     st1, d2, ns2, st2, bias, mult, w, (T*)out, rows, d, groups, eps, write_x)
+#define KLLM_GN1(T, KEEP, CENTRED)                                                                                \
+  hipLaunchKernelGGL((group_norm_add_vec_kernel<T, KEEP, CENTRED>), dim3(n), dim3(kGroupNormThreads), 0, stream, x, d1, \
+                     ns1, st1, d2, ns2, st2, bias, mult, w, norm_bias, (T*)out, rows, d, groups, eps, write_x)
+#define KLLM_GN(T, KEEP)                                                                  \
+  do {                                                                                    \
+    if (norm_bias) KLLM_GN1(T, KEEP, true); else KLLM_GN1(T, KEEP, false);                \
+  } while (0)
     if (out_dtype == DT_F32) {
       if (keep <= 1) KLLM_GN(float, 1); else if (keep <= 2) KLLM_GN(float, 2); else if (keep <= 4) KLLM_GN(float, 4); else KLLM_GN(float, 8);
     } else {
       if (keep <= 1) KLLM_GN(bf16_t, 1); else if (keep <= 2) KLLM_GN(bf16_t, 2); else if (keep <= 4) KLLM_GN(bf16_t, 4); else KLLM_GN(bf16_t, 8);
     }
 #undef KLLM_GN
+#undef KLLM_GN1
     KLLM_CHECK_LAUNCH("group_norm_add");
     return 0;
   }
@@ -272,12 +315,15 @@ extern "C" int kllm_group_norm_add(float* x, const float* d1, int ns1, long st1,
   while (groups * segs < kGroupNormThreads / kWave && d / groups / (2 * segs) >= kWave) segs *= 2;
   const size_t lds = ((size_t)d + (size_t)groups * segs) * sizeof(float);
   KLLM_REQUIRE(lds <= 64 * 1024, "group_norm_add: a row of %d channels in %d groups does not fit into LDS", d, groups);
-  if (out_dtype == DT_F32)
-    hipLaunchKernelGGL(group_norm_add_kernel<float>, dim3(n), dim3(kGroupNormThreads), lds, stream, x, d1, ns1, st1,
-                       d2, ns2, st2, bias, mult, w, (float*)out, rows, d, groups, segs, eps, write_x);
-  else
-    hipLaunchKernelGGL(group_norm_add_kernel<bf16_t>, dim3(n), dim3(kGroupNormThreads), lds, stream, x, d1, ns1, st1,
-                       d2, ns2, st2, bias, mult, w, (bf16_t*)out, rows, d, groups, segs, eps, write_x);
+#define KLLM_GN(T, CENTRED)                                                                                       \
+  hipLaunchKernelGGL((group_norm_add_kernel<T, CENTRED>), dim3(n), dim3(kGroupNormThreads), lds, stream, x, d1, ns1, st1, \
+                     d2, ns2, st2, bias, mult, w, norm_bias, (T*)out, rows, d, groups, segs, eps, write_x)
+  if (out_dtype == DT_F32) {
+    if (norm_bias) KLLM_GN(float, true); else KLLM_GN(float, false);
+  } else {
+    if (norm_bias) KLLM_GN(bf16_t, true); else KLLM_GN(bf16_t, false);
+  }
+#undef KLLM_GN
   KLLM_CHECK_LAUNCH("group_norm_add");
   return 0;
 }

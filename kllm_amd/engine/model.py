@@ -64,7 +64,15 @@ class Model:
             if not 0 <= run.layer < len(self.blocks):
                 raise ValueError(f"schedule entry {i} names layer {run.layer}, the model has "
                                  f"{len(self.blocks)}")
-            need = self.blocks[run.layer].cache_need()
+        needs = [self.blocks[run.layer].cache_need() for run in self.schedule]
+        # a cache that other runs read too is kept for the widest of their windows
+        for i, run in enumerate(self.schedule):
+            j = run.cache_of
+            if (j is not None and 0 <= j < i and isinstance(needs[i], CacheNeed) and isinstance(needs[j], CacheNeed)
+                    and needs[i].alike(needs[j])):
+                needs[j] = needs[j].covering(needs[i])
+        for i, run in enumerate(self.schedule):
+            need = needs[i]
             if isinstance(need, (list, tuple)):
                 # a mixer made of several: every need gets an entry of its own in its group
                 if run.cache_of is not None:
@@ -91,10 +99,9 @@ class Model:
                     raise ValueError(
                         f"schedule entry {i} reads the cache of entry {j}, which must be an "
                         f"earlier entry that writes one")
-                other = self.blocks[self.schedule[j].layer].cache_need()
-                if other.group_key() != need.group_key():
+                if not need.alike(needs[j]):
                     raise ValueError(f"schedule entry {i} cannot read the cache of entry {j}: "
-                                     f"{need} does not fit {other}")
+                                     f"{need} does not fit {needs[j]}")
                 g, e, _ = plan.runs[j]
                 plan.runs.append((g, e, False))
                 continue

@@ -21,7 +21,7 @@ import torch
 DT_F32, DT_BF16 = 0, 1
 GEMM_PLAIN, GEMM_TILED_F32, GEMM_MFMA_BF16, GEMM_SKINNY_BF16, GEMM_GEMV, GEMM_GEMV_LDS, GEMM_MFMA_F32 = 0, 1, 2, 3, 4, 5, 6
 GEMV_BEST_ROWS = 0         # rows up to which they beat the MFMA kernels in bfloat16: none (a step at 1.1B sizes, one token: 1.036 against 0.963 ms)
-ABI_VERSION = 14
+ABI_VERSION = 15
 
 
 class KernelError(RuntimeError):
@@ -112,7 +112,7 @@ def _declare(lib):
         "kllm_command_nargs": [I],
         "kllm_run_commands": [P, L, P, P],
         "kllm_fused_linear_max_parts": [],
-        "kllm_attn_generic": [P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, F, P, I, I, P],
+        "kllm_attn_generic": [P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P, F, P, I, I, P, I, L, L, I, P],
         "kllm_norm_residual": [P, P, I, L, P, P, P, I, I, I, F, P, P, I, P, P, I, I, F, P, P, P, I, L, P, P, F, F, P],
         "kllm_rope_tables_freq": [P, P, P, P, I, I, D, P],
         "kllm_qkv_norm_append": [P, I, L, P, P, P, I, I, I, F, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P],
@@ -136,13 +136,14 @@ def _declare(lib):
         "kllm_calibrate_read": [P, L, P, P],
         "kllm_calibrate_read_workgroups": [],
         "kllm_calibrate_mfma": [I, I, P, P, P],
-        "kllm_attn_decode": [P, P, P, L, P, P, P, P, I, I, I, I, I, I, I, I, I, I, F, P, I, I, P, I, P],
-        "kllm_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, I, F, P, L, I, P, L, I, I, I, P],
+        "kllm_attn_decode": [P, P, P, L, P, P, P, P, I, I, I, I, I, I, I, I, P, I, F, P, I, I, P, I, P, I, L, L, I, P],
+        "kllm_attn_prefill": [P, P, P, P, I, P, P, P, I, I, I, I, I, I, I, P, I, F, P, L, I, P, L, I, I, I, P, I, L, L, I, P],
         "kllm_attn_prefill_slices": [I, I, I],
         "kllm_gemm_act": [P, P, P, I, I, I, I, I, P, P],
         "kllm_add_sinusoid": [P, P, I, I, D, P],
         "kllm_unary_act": [P, I, L, I, P, I, I, I, I, P, P],
-        "kllm_group_norm_add": [P, P, I, L, P, I, L, P, F, P, P, I, P, I, I, I, F, I, P],
+        "kllm_group_norm_add": [P, P, I, L, P, I, L, P, F, P, P, I, P, I, I, I, F, I, P, P],
+        "kllm_soft_cap": [P, L, F, P],
         "kllm_qk_norm_append": [P, I, L, P, P, P, P, F, F, I, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, I, I, P],
         "kllm_delta_prep": [P, I, L, P, P, P, P, I, L, F, F, P, P, I, I, I, I, I, P],
         "kllm_delta_scan_max_dim": [],
@@ -157,7 +158,7 @@ def _declare(lib):
         "kllm_linear_recurrence_scan": [P, P, P, I, L, P, P, L, P, P, P, P, I, I, I, P],
         "kllm_scaled_sum": [P, P, I, L, F, P, I, L, F, L, P],
         "kllm_normed_sum": [P, P, I, L, F, P, P, I, L, F, P, I, I, F, P],
-        "kllm_qkv_conv_append": [P, I, L, I, I, P, I, P, L, I, P, P, I, I, F, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
+        "kllm_qkv_conv_append": [P, I, L, I, I, P, I, P, L, I, P, P, I, I, F, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P, P],
         "kllm_decayed_max_dim": [],
         "kllm_decayed_padded_dim": [I],
         "kllm_decayed_block_numbers": [I, I],
@@ -173,8 +174,8 @@ def _declare(lib):
         "kllm_latent_kv_append": [P, I, L, P, F, P, P, P, P, P, P, I, I, I, I, I, I, L, P],
         "kllm_latent_norm": [P, I, L, L, P, F, P, I, I, I, P],
         "kllm_latent_query": [P, I, L, P, P, P, P, I, I, I, I, I, I, I, P],
-        "kllm_attn_latent": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, L, I, P],
-        "kllm_latent_out": [P, P, P, I, L, L, P, I, I, I, I, I, P],
+        "kllm_attn_latent": [P, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P, L, I, I, P],
+        "kllm_latent_out": [P, P, P, I, L, L, P, I, I, I, I, I, I, P],
     }
     for name, args in sigs.items():
         fn = getattr(lib, name)
@@ -200,7 +201,7 @@ LAUNCHING = ("kllm_embed", "kllm_add_rmsnorm", "kllm_rope_tables", "kllm_rope_ap
              "kllm_conv_state_update", "kllm_gated_delta_prep", "kllm_gated_delta_scan", "kllm_linear_recurrence_prep",
              "kllm_linear_recurrence_scan", "kllm_latent_kv_append", "kllm_latent_norm", "kllm_latent_query", "kllm_attn_latent",
              "kllm_latent_out", "kllm_scaled_sum", "kllm_normed_sum", "kllm_qkv_conv_append", "kllm_decayed_prep",
-             "kllm_decayed_scan", "kllm_decayed_out", "kllm_decayed_step", "kllm_token_gate")
+             "kllm_decayed_scan", "kllm_decayed_out", "kllm_decayed_step", "kllm_token_gate", "kllm_soft_cap")
 DYNAMIC_ARGS = {"kllm_attn_prefill": (19, 20)}     # arguments that may be a StepValue
 STRUCT_ARGS = {"kllm_gemv_plain": (7,), "kllm_gemv_swiglu": (8,), "kllm_gemv_rope_append": (17,),
                "kllm_fused_linear": (2,)}
@@ -1067,6 +1068,36 @@ def _slopes(slopes, n_heads, who):
     return _ptr(slopes, who + " slopes", torch.float32, True)
 
 
+_zero_sinks = {}
+
+
+def _sinks(sink, n_heads, device, who):
+    """Pointer of the per-head scores of a key without a value that joins every softmax (float32
+    [heads]; True: a score of 0 for every head), or null for none."""
+    if sink is None or sink is False:
+        return 0
+    if sink is True:
+        key = (device, n_heads)
+        if key not in _zero_sinks:
+            _zero_sinks[key] = torch.zeros(n_heads, dtype=torch.float32, device=device)
+        sink = _zero_sinks[key]
+    if sink.numel() != n_heads:
+        raise KernelError(f"{who}: {sink.numel()} sinks for {n_heads} heads")
+    return _ptr(sink, who + " sinks", torch.float32)
+
+
+def _out_gate(gate, n, n_heads, value_dim, who):
+    """The arguments of a gate on attention's output: ``gate`` None, or ``Columns`` of float32 sums with
+    as many columns a head as are gated (at most the value's width)."""
+    if gate is None:
+        return 0, 0, 0, 0, 0
+    width = gate.width // n_heads
+    if width * n_heads != gate.width or not 0 < width <= value_dim:
+        raise KernelError(f"{who}: a gate of {gate.width} columns for {n_heads} heads of {value_dim}")
+    addr, nsplit, stride, row = gate.place(n, who + " gate")
+    return addr + 4 * gate.first, nsplit, stride, row, width
+
+
 def paged_cache_fits(cache, n_kv_heads, page_size, head_dim, value_dim):
     """Whether ``cache`` is a pool of pages for keys of ``head_dim`` and values of ``value_dim``:
     [pages, 2, KV, page_size * head_dim] where the two are equal, or flat pages of
@@ -1078,13 +1109,16 @@ def paged_cache_fits(cache, n_kv_heads, page_size, head_dim, value_dim):
 
 
 def attn_generic(q, out, cache, positions, span_of_token, block_table, page_size, n_heads,
-                 n_kv_heads, head_dim, window, scale, slopes=None, value_dim=None, chunk=0, sink=False, keep_first=0):
+                 n_kv_heads, head_dim, window, scale, slopes=None, value_dim=None, chunk=0, sink=False, keep_first=0,
+                 gate=None):
     """``keep_first`` > 0: the first keep_first positions of a request stay readable behind the
     window.  ``slopes`` (here and in the other attention wrappers): float32 [heads] or None; slopes[h]
     times the distance from the query to the key is taken off head h's scaled scores.
     ``value_dim``: width of a value (default: the key's); ``chunk`` > 0: the query at position p
-    reads no key before p - p % chunk; ``sink``: the softmax's denominator has one more term,
-    exp(0)."""
+    reads no key before p - p % chunk; ``sink``: the softmax's denominator has one more term:
+    exp(0) for True, exp(sink[h]) for a float32 tensor [heads], neither scaled nor biased.  ``gate``
+    (``Columns`` of float32 sums, as many a head as the value's width or, for padded values, fewer):
+    the output is multiplied by its logistic function element by element."""
     n = q.shape[0]
     vd = head_dim if value_dim is None else int(value_dim)
     if (tuple(q.shape) != (n, n_heads * head_dim) or tuple(out.shape) != (n, n_heads * vd)
@@ -1098,8 +1132,9 @@ def attn_generic(q, out, cache, positions, span_of_token, block_table, page_size
         _ptr(positions, "attn positions", torch.int32),
         _ptr(span_of_token, "attn span_of_token", torch.int32),
         _ptr(block_table, "attn block_table", torch.int32), block_table.shape[1], page_size, n,
-        n_heads, n_kv_heads, head_dim, vd, int(window), int(chunk), int(bool(sink)), float(scale),
-        _slopes(slopes, n_heads, "attn_generic"), dtype_code(q.dtype), int(keep_first), _stream())
+        n_heads, n_kv_heads, head_dim, vd, int(window), int(chunk), _sinks(sink, n_heads, q.device, "attn_generic"),
+        float(scale), _slopes(slopes, n_heads, "attn_generic"), dtype_code(q.dtype), int(keep_first),
+        *_out_gate(gate, n, n_heads, vd, "attn_generic"), _stream())
 
 
 GENERIC_MAX_PAGE_SIZE = 256     # pages of the kernel that takes every size
@@ -1153,7 +1188,7 @@ def attn_prefill_slices(n_tiles, n_heads, head_dim, dtype=torch.bfloat16) -> int
 
 def attn_prefill(q, out, cache, query_tiles, n_tiles, span_start, span_pos, block_table, page_size,
                  n_heads, n_kv_heads, head_dim, window, scale, keys_total=0, keys_longest=0, part=None,
-                 nslices=None, slopes=None, chunk=0, sink=False, keep_first=0):
+                 nslices=None, slopes=None, chunk=0, sink=False, keep_first=0, gate=None):
     """query_tiles [n_tiles, 2] int32: (first token row, span) of each block of up to
     PREFILL_QUERY_BLOCK consecutive tokens of one span.  ``keys_total`` and
     ``keys_longest``: how many keys the blocks read, all together and the longest block
@@ -1180,17 +1215,17 @@ def attn_prefill(q, out, cache, query_tiles, n_tiles, span_start, span_pos, bloc
         _ptr(query_tiles, "attn query_tiles", torch.int32), n_tiles,
         _ptr(span_start, "attn span_start", torch.int32), _ptr(span_pos, "attn span_pos", torch.int32),
         _ptr(block_table, "attn block_table", torch.int32), block_table.shape[1], page_size,
-        n_heads, n_kv_heads, head_dim, int(window), int(chunk), int(bool(sink)), int(keep_first), float(scale),
-        _slopes(slopes, n_heads, "attn_prefill"),
+        n_heads, n_kv_heads, head_dim, int(window), int(chunk), _sinks(sink, n_heads, q.device, "attn_prefill"),
+        int(keep_first), float(scale), _slopes(slopes, n_heads, "attn_prefill"),
         keys_total if type(keys_total) is StepValue else int(keys_total),
         keys_longest if type(keys_longest) is StepValue else int(keys_longest),
         _ptr(part, "attn part", torch.float32, True) if nslices > 1 else 0, need, nslices, n,
-        dtype_code(q.dtype), _stream())
+        dtype_code(q.dtype), *_out_gate(gate, n, n_heads, head_dim, "attn_prefill"), _stream())
 
 
 def attn_decode(q, out, part, cache, positions, span_of_token, block_table, page_size, n_heads,
                 n_kv_heads, head_dim, window, scale, nslices, token_list=None, n_listed=0, slopes=None, chunk=0,
-                sink=False, keep_first=0):
+                sink=False, keep_first=0, gate=None):
     n = q.shape[0]
     if (tuple(q.shape) != (n, n_heads * head_dim) or tuple(out.shape) != tuple(q.shape)
             or q.dtype != cache.dtype or out.dtype != q.dtype):
@@ -1203,10 +1238,11 @@ def attn_decode(q, out, part, cache, positions, span_of_token, block_table, page
         part.numel(), _ptr(cache, "attn cache"), _ptr(positions, "attn positions", torch.int32),
         _ptr(span_of_token, "attn span_of_token", torch.int32),
         _ptr(block_table, "attn block_table", torch.int32), block_table.shape[1], page_size, n,
-        n_heads, n_kv_heads, head_dim, int(window), int(chunk), int(bool(sink)), int(keep_first), float(scale),
-        _slopes(slopes, n_heads, "attn_decode"),
+        n_heads, n_kv_heads, head_dim, int(window), int(chunk), _sinks(sink, n_heads, q.device, "attn_decode"),
+        int(keep_first), float(scale), _slopes(slopes, n_heads, "attn_decode"),
         int(nslices), dtype_code(q.dtype),
-        _ptr(token_list, "attn token_list", torch.int32, True), int(n_listed), _stream())
+        _ptr(token_list, "attn token_list", torch.int32, True), int(n_listed),
+        *_out_gate(gate, n, n_heads, head_dim, "attn_decode"), _stream())
 
 
 def sample(out, logits, temperature=None, uniform=None):
@@ -1272,10 +1308,12 @@ def gemm_act(x, w, h, act, params=None):
 
 
 def group_norm_add(x, deltas=(), bias=None, mult=1.0, weight=None, out=None, rows=None, groups=1, eps=0.0,
-                   write_x=None):
+                   write_x=None, norm_bias=None):
     """x [N, d] float32; v = x + mult * (the deltas' slices summed + bias), written back to x
     (unless ``rows`` selects rows to read); out [n, d] = v normalised in ``groups`` groups of
-    channels, times weight.  ``deltas``: up to two float32 tensors [N, d] or [nsplit, N, d]."""
+    channels, times weight.  ``deltas``: up to two float32 tensors [N, d] or [nsplit, N, d].  With
+    ``norm_bias`` [d] (one group) the norm is taken around the row's mean, and the bias is added:
+    out = (v - mean) / sqrt(mean((v - mean)^2) + eps) * weight + norm_bias."""
     N, d = x.shape
     deltas = [t for t in deltas if t is not None]
     if len(deltas) > 2:
@@ -1287,6 +1325,8 @@ def group_norm_add(x, deltas=(), bias=None, mult=1.0, weight=None, out=None, row
         raise KernelError("group_norm_add: output or weight shape does not fit")
     if bias is not None and bias.numel() != d:
         raise KernelError("group_norm_add: bias does not fit")
+    if norm_bias is not None and (norm_bias.numel() != d or int(groups) != 1):
+        raise KernelError("group_norm_add: the norm's bias does not fit")
     args = []
     for t in deltas + [None] * (2 - len(deltas)):
         if t is None:
@@ -1298,7 +1338,13 @@ def group_norm_add(x, deltas=(), bias=None, mult=1.0, weight=None, out=None, row
             _ptr(bias, "group_norm_add bias", torch.float32, True), float(mult),
             _ptr(weight, "group_norm_add weight", torch.float32, True), _ptr(out, "group_norm_add out", None, True),
             dtype_code(out.dtype) if out is not None else DT_F32, _ptr(rows, "group_norm_add rows", torch.int32, True),
-            n, d, int(groups), float(eps), int(bool(write_x)), _stream())
+            n, d, int(groups), float(eps), int(bool(write_x)),
+            _ptr(norm_bias, "group_norm_add norm bias", torch.float32, True), _stream())
+
+
+def soft_cap(x, cap):
+    """x = cap * tanh(x / cap), float32, in place."""
+    _launch("kllm_soft_cap", "soft_cap", _ptr(x, "soft_cap x", torch.float32), x.numel(), float(cap), _stream())
 
 
 def qk_norm_append(qk, q_out, cache, positions, span_of_token, block_table, page_size, n_heads, n_kv_heads,
@@ -1820,19 +1866,24 @@ class Columns:
 
 def qkv_conv_append(qkv, conv_w, taps, state, conv_offset, single, q_out, cache, positions, span_of_token, slots, span_start,
                     span_pos, block_table, page_size, n_heads, n_kv_heads, head_dim, value_dim, width, cos=None, sin=None,
-                    rotary_dim=0, interleaved=False, v_scale=1.0):
+                    rotary_dim=0, interleaved=False, v_scale=1.0, bias=None):
     """``qkv`` (Columns): q (H head_dim) | k (KV head_dim) | v (KV value_dim).  Each channel passes a causal
     convolution (conv_w [channels, taps]; earlier inputs from the state's field at ``conv_offset``), the
     first ``rotary_dim`` elements of every query and key head turn (cos, sin [n, rotary_dim / 2]);
     writes q_out [n, H * width] and appends keys and values (times ``v_scale``) to pages whose slots hold
     ``width`` elements, zeros beyond a head's own.  ``single``: every span is one token, and the state
-    takes the new inputs in the same launch (otherwise ``conv_state_update`` follows)."""
+    takes the new inputs in the same launch (otherwise ``conv_state_update`` follows).  Without weights
+    (``conv_w`` None, one tap) nothing is convolved and ``bias`` [channels] is added instead; without a
+    cache (None, no KV heads) there are queries only."""
     n = q_out.shape[0]
     C = (n_heads + n_kv_heads) * head_dim + n_kv_heads * value_dim
     addr, nsplit, stride, row = qkv.place(n, "qkv_conv_append")
-    if (qkv.width < C or tuple(conv_w.shape) != (C, taps) or q_out.shape[1] != n_heads * width
-            or not paged_cache_fits(cache, n_kv_heads, page_size, width, width) or cache.dtype != q_out.dtype):
-        raise KernelError(f"qkv_conv_append: sums, weights, q_out or cache {tuple(cache.shape)} do not fit")
+    if (qkv.width < C or (conv_w is not None and tuple(conv_w.shape) != (C, taps)) or q_out.shape[1] != n_heads * width
+            or (bias is not None and bias.numel() != C) or (conv_w is None and taps != 1)):
+        raise KernelError("qkv_conv_append: sums, weights, bias or q_out do not fit")
+    if (cache is None) != (n_kv_heads == 0) or (cache is not None and (
+            not paged_cache_fits(cache, n_kv_heads, page_size, width, width) or cache.dtype != q_out.dtype)):
+        raise KernelError(f"qkv_conv_append: cache {None if cache is None else tuple(cache.shape)} does not fit")
     if positions.numel() < n or span_of_token.numel() < n:
         raise KernelError("qkv_conv_append: index arrays are too short")
     rot = int(rotary_dim) if cos is not None else 0
@@ -1843,13 +1894,14 @@ def qkv_conv_append(qkv, conv_w, taps, state, conv_offset, single, q_out, cache,
         raise KernelError("qkv_conv_append: the state is too short")
     F32, I32 = torch.float32, torch.int32
     _launch("kllm_qkv_conv_append", "qkv_conv_append", addr, nsplit, stride, row, qkv.first,
-            _ptr(conv_w, "conv weights", F32), int(taps), st, per_slot, 1 if single else 0,
+            _ptr(conv_w, "conv weights", F32, True), int(taps), st, per_slot, 1 if single else 0,
             _ptr(cos, "conv cos", F32, True), _ptr(sin, "conv sin", F32, True), rot, int(bool(interleaved)), float(v_scale),
-            _ptr(q_out, "conv q_out"), _ptr(cache, "conv cache"), _ptr(positions, "conv positions", I32),
+            _ptr(q_out, "conv q_out"), _ptr(cache, "conv cache", None, True), _ptr(positions, "conv positions", I32),
             _ptr(span_of_token, "conv span_of_token", I32), _ptr(slots, "conv slots", I32),
             _ptr(span_start, "conv span_start", I32), _ptr(span_pos, "conv span_pos", I32),
             _ptr(block_table, "conv block_table", I32), block_table.shape[1], int(page_size), n, int(n_heads),
-            int(n_kv_heads), int(head_dim), int(value_dim), int(width), dtype_code(q_out.dtype), _stream())
+            int(n_kv_heads), int(head_dim), int(value_dim), int(width), dtype_code(q_out.dtype),
+            _ptr(bias, "conv bias", F32, True), _stream())
 
 
 def decayed_max_dim() -> int:
@@ -2098,11 +2150,12 @@ def latent_query(q, w_uk, cos, sin, out, heads, dim, rot_dim, rank, transposed=F
 LATENT_BLOCK_FROM = 64      # tokens of a step from which four tokens share a workgroup and its tiles of keys
 
 
-def attn_latent_slices(n, heads, rank, dtype=torch.bfloat16) -> int:
+def attn_latent_slices(n, heads, rank, dtype=torch.bfloat16, window=0) -> int:
     """Workgroups that share out the keys of a token and 16 heads (their results are merged in
     the same call): as many as bring a step's workgroups to about two a CU, for steps of few
     tokens; 1 where the kernel on the matrix cores does not run; 0 for steps of many tokens: there
-    a workgroup takes four tokens, whose keys pass through LDS once for the four.  Does not depend on any context
+    a workgroup takes four tokens, whose keys pass through LDS once for the four.  A ``window`` bounds a
+    token's keys: a slice has 128 of them at least.  Does not depend on any context
     length, so a recorded step can be replayed as contexts grow."""
     if dtype != torch.bfloat16 or rank % 16 or rank > 512:
         return 1
@@ -2110,16 +2163,17 @@ def attn_latent_slices(n, heads, rank, dtype=torch.bfloat16) -> int:
         return 0
     groups = n * ((heads + 15) // 16)
     slices = 1
-    while slices < 32 and groups * slices * 2 <= 2 * device_cus():
+    most = min(32, -(-(window + 31) // 128)) if window else 32
+    while slices < most and groups * slices * 2 <= 2 * device_cus():
         slices *= 2
     return slices
 
 
 def attn_latent(q, out, cache, positions, span_of_token, block_table, page_size, heads, row, rank, scale, plain=False,
-                part=None, nslices=1):
+                part=None, nslices=1, window=0):
     """Causal attention of q [n, H row] over cached rows of ``row`` elements whose first ``rank``
     are also the values (a page: its rows, then the first ``rank`` elements once more as
-    [rank][slot]): out [n, H rank].  ``plain``: the kernel for every size, also where the one on
+    [rank][slot]): out [n, H rank].  ``window`` > 0: of the last ``window`` rows only.  ``plain``: the kernel for every size, also where the one on
     the matrix cores fits."""
     n = q.shape[0]
     if (tuple(q.shape) != (n, heads * row) or tuple(out.shape) != (n, heads * rank) or q.dtype != cache.dtype
@@ -2132,18 +2186,19 @@ def attn_latent(q, out, cache, positions, span_of_token, block_table, page_size,
             _ptr(span_of_token, "attn_latent span_of_token", I32), _ptr(block_table, "attn_latent block_table", I32),
             block_table.shape[1], int(page_size), n, int(heads), int(row), int(rank), float(scale), dtype_code(q.dtype),
             int(bool(plain)), _ptr(part, "attn_latent part", torch.float32, True) if nslices > 1 else 0,
-            part.numel() if nslices > 1 else 0, int(nslices), _stream())
+            part.numel() if nslices > 1 else 0, int(nslices), int(window), _stream())
 
 
-def latent_out(attended, w_uv, out, heads, vdim, rank, gate=None, gate_column=0):
+def latent_out(attended, w_uv, out, heads, vdim, rank, gate=None, gate_column=0, gate_by_head=False):
     """out [n, H vdim] = per head w_uv ([H vdim, rank]) times attended [n, H rank], times sigmoid of
-    columns gate_column .. + H vdim of the float32 sums ``gate`` (None: no gate)."""
+    columns gate_column .. + H vdim of the float32 sums ``gate`` (None: no gate), or of columns
+    gate_column .. + H, one a head (``gate_by_head``)."""
     n = out.shape[0]
-    addr, nsplit, stride, cols = _columns(gate, gate_column, heads * vdim, "latent_out") if gate is not None else (0, 0, 0, 0)
+    addr, nsplit, stride, cols = _columns(gate, gate_column, heads * (1 if gate_by_head else vdim), "latent_out") if gate is not None else (0, 0, 0, 0)
     if (tuple(attended.shape) != (n, heads * rank) or tuple(out.shape) != (n, heads * vdim)
             or tuple(w_uv.shape) != (heads * vdim, rank) or w_uv.dtype != out.dtype or attended.dtype != out.dtype
             or (gate is not None and gate.shape[-2] != n)):
         raise KernelError("latent_out: shapes or dtypes do not fit")
     _launch("kllm_latent_out", "latent_out", _ptr(attended, "latent attended"), _ptr(w_uv, "latent w_uv"),
             addr, nsplit, stride, cols, _ptr(out, "latent out"), n, int(heads), int(vdim), int(rank),
-            dtype_code(out.dtype), _stream())
+            dtype_code(out.dtype), int(bool(gate_by_head)), _stream())

@@ -14,7 +14,8 @@ head h's scaled scores lose 2^(-b (h+1) / heads) times the distance from the
 query to the key), ``chunk`` (0: none; c: a chunked mask, the query at position
 p reads no key before p - p % c, chunks counted from the request's position 0),
 ``sink`` (False; True: the softmax's denominator has one more term, exp(0): a
-key whose score is 0 and that has no value), ``value_dim`` (width of a value;
+key whose score is 0 and that has no value; "learned": exp of a number per head, a
+tensor of the part, for parts that have one), ``value_dim`` (width of a value;
 default: the key's), ``keep_first`` (with a window: the first ``keep_first``
 positions of a request stay readable behind it, at their true positions).
 Tensors: ``<prefix>.{q,k,v,o}_proj.weight``.  The three input projections are
@@ -46,6 +47,8 @@ class CausalSelfAttention(Part):
     SHORT_SPAN = 4
     QUERY_BLOCK = K.PREFILL_QUERY_BLOCK
     FAST_KERNELS_OFF = False
+    learns_sinks = False      # whether the part has a tensor for ``sink`` "learned"
+    pads_heads = False        # whether the pages' slots may be wider than the heads
 
     def step_lists(self, starts, lens):
         short, blocks = [], []
@@ -83,7 +86,10 @@ class CausalSelfAttention(Part):
         self.head_dim = int(self.param("head_dim"))
         self.window = int(self.param("window", 0) or 0)
         self.chunk = int(self.param("chunk", 0) or 0)
-        self.sink = bool(self.param("sink", False))
+        self.sink = self.param("sink", False)
+        self.sinks = None           # float32 [heads] on the device once bound: the score of a key without a value
+        if self.sink not in (False, True, None) and not (self.sink == "learned" and self.learns_sinks):
+            raise ValueError(f"attention: sink {self.sink!r} is not built for this part")
         self.value_dim = int(self.param("value_dim", None) or self.head_dim)
         self.keep_first = int(self.param("keep_first", 0) or 0) if self.window else 0
         if self.chunk < 0 or self.keep_first < 0 or not 0 < self.value_dim <= 256:
@@ -95,7 +101,7 @@ class CausalSelfAttention(Part):
         self.own_kv = bool(self.param("own_kv", True))
         if self.heads % self.kv_heads:
             raise ValueError(f"attention: {self.heads} heads are not a multiple of {self.kv_heads} KV heads")
-        if self.head_dim % 2 or self.head_dim > 256:
+        if (self.head_dim % 2 and not self.pads_heads) or self.head_dim > 256:
             raise ValueError(f"attention: head_dim {self.head_dim} must be even and at most 256")
         pos = self.param("position", None)
         self.position = runtime.shared_part("position", pos) if pos is not None else None
@@ -129,9 +135,29 @@ class CausalSelfAttention(Part):
         return specs
 
     def _bind_slopes(self):
+        if self.sink is True:
+            self.sinks = torch.zeros(self.heads, dtype=torch.float32, device=self.runtime.device)
         if self.slope_bits is not None:
             values = [2.0 ** (-self.slope_bits * (h + 1) / self.heads) for h in range(self.heads)]
             self.slopes = torch.tensor(values, dtype=torch.float32, device=self.runtime.device)
+
+    # ---- parts that ``pads_heads``: pages hold one width for keys and values, the smallest that the
+    # kernels on the matrix cores take for both (the rest of a slot is zero)
+    def _pad_heads(self):
+        self.key_dim, self.val_dim = self.head_dim, self.value_dim
+        widest = max(self.key_dim, self.val_dim)
+        self.width = next(w for w in K.PREFILL_HEAD_DIMS if w >= widest)
+        # the rest of this class sees heads of the pages' width
+        self.head_dim = self.value_dim = self.width
+        self.q_dim = self.out_dim = self.heads * self.width
+        self.kv_dim = self.kv_heads * self.width
+
+    def _padded_output(self, w_o):
+        """The output projection with columns of zeros where a head's output is padding."""
+        if self.width == self.val_dim:
+            return w_o
+        by_head = w_o.reshape(self.hidden, self.heads, self.val_dim)
+        return torch.nn.functional.pad(by_head, (0, self.width - self.val_dim)).reshape(self.hidden, -1).contiguous()
 
     def bind(self, weights):
         self._bind_slopes()
@@ -219,12 +245,13 @@ class CausalSelfAttention(Part):
                 return normed
         return linear(ctx, out, self.w_o, "attn.proj")
 
-    def attend(self, ctx, q, out, cache):
+    def attend(self, ctx, q, out, cache, gate=None):
         """Choose the attention kernels by the spans' lengths: tokens of short
         spans (decode tokens) go to the kernel that splits a token's keys over
         many waves, longer spans to the prompt kernel in blocks of 128 queries
         (both on the matrix cores, in bfloat16 or with 32-bit operands); sizes
-        those kernels do not take go to the kernel that takes every size."""
+        those kernels do not take go to the kernel that takes every size.  ``gate``
+        (``K.Columns`` of sums): its logistic function multiplies the output."""
         mode = self.runtime.options.get("attention", "auto")
         if q.dtype == torch.bfloat16:
             fast = cache.page_size % 16 == 0 and self.head_dim in K.DECODE_HEAD_DIMS
@@ -238,8 +265,8 @@ class CausalSelfAttention(Part):
         if not fast:
             K.attn_generic(q, out, cache.pages, ctx.positions, ctx.span_of_token, cache.block_table,
                            cache.page_size, self.heads, self.kv_heads, self.head_dim, self.window,
-                           self.scale, slopes=self.slopes, value_dim=self.value_dim, chunk=self.chunk, sink=self.sink,
-                           keep_first=self.keep_first)
+                           self.scale, slopes=self.slopes, value_dim=self.value_dim, chunk=self.chunk, sink=self.sinks,
+                           keep_first=self.keep_first, gate=gate)
             return
         n = q.shape[0]
         short = ctx.lists.get("attention.spans.short")
@@ -247,10 +274,10 @@ class CausalSelfAttention(Part):
         n_short = short.numel() if short is not None else 0
         n_blocks = blocks.numel() // 2 if blocks is not None else 0
         if n_short + n_blocks == 0 or (n_blocks and not prompt_ok):   # a context built by hand may carry no lists
-            self._decode(ctx, q, out, cache, None, n)   # token by token
+            self._decode(ctx, q, out, cache, None, n, gate)   # token by token
             return
         if n_short:
-            self._decode(ctx, q, out, cache, None if n_short == n else short, n_short)
+            self._decode(ctx, q, out, cache, None if n_short == n else short, n_short, gate)
         if n_blocks:
             total, longest = self._keys_read(ctx)
             part = None
@@ -261,8 +288,8 @@ class CausalSelfAttention(Part):
             K.attn_prefill(q, out, cache.pages, blocks, n_blocks, ctx.span_start,
                            ctx.span_pos, cache.block_table, cache.page_size, self.heads,
                            self.kv_heads, self.head_dim, self.window, self.scale, total, longest, part=part,
-                           nslices=slices, slopes=self.slopes, chunk=self.chunk, sink=self.sink,
-                           keep_first=self.keep_first)
+                           nslices=slices, slopes=self.slopes, chunk=self.chunk, sink=self.sinks,
+                           keep_first=self.keep_first, gate=gate)
 
     def _keys_read(self, ctx):
         """The step's key counts (see ``step_values``), as the engine worked them out for this
@@ -273,7 +300,7 @@ class CausalSelfAttention(Part):
         own = self.step_values(ctx.h_span_start, ctx.h_span_len, ctx.h_span_pos)
         return own["keys_total"], own["keys_longest"]
 
-    def _decode(self, ctx, q, out, cache, token_list, count):
+    def _decode(self, ctx, q, out, cache, token_list, count, gate=None):
         n = q.shape[0]
         # The block table's width bounds the keys of the step's longest request.  It is rounded up
         # to a power of two of pages (from 8), as recorded steps round theirs: a step then cuts
@@ -291,8 +318,8 @@ class CausalSelfAttention(Part):
         part = ctx.buf("attn.part", (n * self.heads * nslices * (self.head_dim + 2),), torch.float32)
         K.attn_decode(q, out, part, cache.pages, ctx.positions, ctx.span_of_token, cache.block_table,
                       cache.page_size, self.heads, self.kv_heads, self.head_dim, self.window,
-                      self.scale, nslices, token_list, count, slopes=self.slopes, chunk=self.chunk, sink=self.sink,
-                      keep_first=self.keep_first)
+                      self.scale, nslices, token_list, count, slopes=self.slopes, chunk=self.chunk, sink=self.sinks,
+                      keep_first=self.keep_first, gate=gate)
 
 
 @register_part("mixer", "attention_keys_as_values")
@@ -570,7 +597,7 @@ class ConvolvedAttention(CausalSelfAttention):
     fills_sink = False
     shares_input = True       # its input product may be a part of a larger one (``sums``)
     folds_scale = True        # a factor on its output (``out_scale``) is a factor on its values
-    WIDTHS = K.PREFILL_HEAD_DIMS
+    pads_heads = True
     MAX_TAPS = 16
 
     def __init__(self, spec, runtime):
@@ -580,13 +607,7 @@ class ConvolvedAttention(CausalSelfAttention):
         self.taps = int(self.param("taps"))
         if not 1 <= self.taps <= self.MAX_TAPS:
             raise ValueError(f"attention_conv: a convolution of {self.taps} taps is not built (1 to {self.MAX_TAPS})")
-        self.key_dim, self.val_dim = self.head_dim, self.value_dim
-        widest = max(self.key_dim, self.val_dim)
-        self.width = next(w for w in self.WIDTHS if w >= widest)
-        # the base class sees heads of the pages' width
-        self.head_dim = self.value_dim = self.width
-        self.q_dim = self.out_dim = self.heads * self.width
-        self.kv_dim = self.kv_heads * self.width
+        self._pad_heads()
         self.channels = (self.heads + self.kv_heads) * self.key_dim + self.kv_heads * self.val_dim
         self.out_scale = 1.0
         self.conv = None
@@ -603,10 +624,7 @@ class ConvolvedAttention(CausalSelfAttention):
         w = lambda n: weights[self.tensor_name(n)]
         self.w_in = torch.cat([w(t + ".weight") for t in ("q", "k", "v")], dim=0).contiguous()
         self.conv = torch.cat([w(t + ".conv") for t in ("q", "k", "v")], dim=0).contiguous()
-        self.w_o = w("o.weight")
-        if self.width != self.val_dim:       # columns of zeros where a head's output is padding
-            by_head = self.w_o.reshape(self.hidden, self.heads, self.val_dim)
-            self.w_o = torch.nn.functional.pad(by_head, (0, self.width - self.val_dim)).reshape(self.hidden, -1).contiguous()
+        self.w_o = self._padded_output(w("o.weight"))
         self._tiled = {"in": tiled_copy(self.runtime, self.w_in, K.LINEAR_PARTS),
                        "o": tiled_copy(self.runtime, self.w_o, K.LINEAR_PARTS)}
 
@@ -650,4 +668,82 @@ class ConvolvedAttention(CausalSelfAttention):
                                 ctx.span_pos, ctx.n_spans)
         out = ctx.buf("attn.out", (n, self.out_dim), dtype)
         self.attend(ctx, q, out, pages)
+        return decode_linear(ctx, out, self.w_o, "attn.proj", self._tiled.get("o"))
+
+
+@register_part("mixer", "attention_bias")
+class BiasedAttention(CausalSelfAttention):
+    """Attention whose projections have biases and whose output passes a gate: q = W_q h + b_q, k = W_k h
+    + b_k, v = W_v h + b_v, no rotation; scores ((q . k) * ``scale``, less the distance bias), mask
+    (``window``, ``chunk``), ``sink`` and the kernels are the base class's, and with ``sink``
+    "learned" the softmax's extra term is exp of a number per head.  With ``gate`` the concatenated
+    heads are multiplied element by element by the logistic function of W_g h, where attention's
+    kernels write their output.  The output projection's bias is left to whoever adds the output to
+    the stream (``out_bias``).  Values may have a width of their own.
+
+    With ``own_kv`` False the part has no k and v: it reads the keys and values that another run cached.
+
+    Pages hold one width for keys and values, the smallest that the kernels on the matrix cores take
+    for both (the rest of a slot is zero); the output projection's columns are padded likewise.
+
+    Parameters beyond the base class's: ``gate`` (default False).
+    Tensors: ``<prefix>.{q,k,v,g,o}.weight``, ``.{q,k,v,o}.bias``, ``.sink`` [heads]."""
+    takes_normed = False
+    fills_sink = False
+    learns_sinks = True
+    pads_heads = True
+
+    def __init__(self, spec, runtime):
+        super().__init__(spec, runtime)
+        if self.position is not None or self.keep_first:
+            raise ValueError("attention_bias: takes no position part and keeps no first positions")
+        self.gated = bool(self.param("gate", False))
+        self._pad_heads()
+        own = self.kv_heads if self.own_kv else 0
+        self.rows = {"q": self.heads * self.key_dim}
+        if own:
+            self.rows.update(k=own * self.key_dim, v=own * self.val_dim)
+        self.channels = sum(self.rows.values())
+        self.gate_dim = self.heads * self.val_dim
+        self.bias = self.out_bias = None
+
+    def weight_specs(self):
+        d, name = self.hidden, self.tensor_name
+        specs = [WeightSpec(name(t + ".weight"), (n, d)) for t, n in self.rows.items()]
+        specs += [WeightSpec(name(t + ".bias"), (n,), "vector") for t, n in self.rows.items()]
+        if self.gated:
+            specs.append(WeightSpec(name("g.weight"), (self.gate_dim, d)))
+        if self.sink == "learned":
+            specs.append(WeightSpec(name("sink"), (self.heads,), "vector"))
+        return specs + [WeightSpec(name("o.weight"), (d, self.gate_dim)), WeightSpec(name("o.bias"), (d,), "vector")]
+
+    def bind(self, weights):
+        self._bind_slopes()
+        w = lambda n: weights[self.tensor_name(n)]
+        # one product for everything that reads the layer's input: queries | keys | values | gate
+        self.w_in = torch.cat([w(t + ".weight") for t in [*self.rows] + (["g"] if self.gated else [])], dim=0).contiguous()
+        self.bias = torch.cat([w(t + ".bias") for t in self.rows]).contiguous()
+        if self.sink == "learned":
+            self.sinks = w("sink")
+        self.w_o, self.out_bias = self._padded_output(w("o.weight")), w("o.bias")
+        # second copies for decode batches, in the order that kernel reads them
+        self._tiled = {"in": tiled_copy(self.runtime, self.w_in, K.LINEAR_PARTS),
+                       "o": tiled_copy(self.runtime, self.w_o, K.LINEAR_PARTS)}
+
+    def flops(self, tokens, keys_read=0.0):
+        return (2.0 * tokens * (self.w_in.numel() + self.hidden * self.gate_dim)
+                + 2.0 * self.heads * (self.key_dim + self.val_dim) * keys_read)
+
+    def forward(self, ctx, xn, cache):
+        n = xn.shape[0]
+        if self.own_kv != bool(cache.write):
+            raise ValueError("attention_bias: a run must write its cache exactly when it has k and v projections")
+        sums = decode_linear(ctx, xn, self.w_in, "attn.qkvg", self._tiled.get("in"))
+        q = ctx.buf("attn.q", (n, self.q_dim), self.runtime.dtype)
+        K.qkv_conv_append(K.Columns(sums, 0, self.channels), None, 1, None, 0, ctx.all_decode, q,
+                          cache.pages if self.own_kv else None, ctx.positions, ctx.span_of_token, ctx.slots, ctx.span_start,
+                          ctx.span_pos, cache.block_table, cache.page_size, self.heads, self.kv_heads if self.own_kv else 0,
+                          self.key_dim, self.val_dim, self.width, bias=self.bias)
+        out = ctx.buf("attn.out", (n, self.out_dim), self.runtime.dtype)
+        self.attend(ctx, q, out, cache, gate=K.Columns(sums, self.channels, self.gate_dim) if self.gated else None)
         return decode_linear(ctx, out, self.w_o, "attn.proj", self._tiled.get("o"))

@@ -79,6 +79,9 @@ class LinearHead(Part):
         super().__init__(spec, runtime)
         self.vocab = int(self.param("vocab"))
         self.hidden = int(self.param("hidden"))
+        # a soft cap on the logits: z becomes cap * tanh(z / cap) (None: none)
+        cap = self.param("soft_cap", None)
+        self.soft_cap = float(cap) if cap is not None else None
         self.weight = None
 
     def weight_specs(self):
@@ -89,4 +92,7 @@ class LinearHead(Part):
         self._tiled = {"w": tiled_copy(self.runtime, self.weight, K.LINEAR_PARTS)}   # for decode batches
 
     def forward(self, ctx, xn_rows):
-        return linear(ctx, xn_rows, self.weight, "logits", split=False, w_tiled=self._tiled.get("w"))
+        logits = linear(ctx, xn_rows, self.weight, "logits", split=False, w_tiled=self._tiled.get("w"))
+        if self.soft_cap is not None:
+            K.soft_cap(logits, self.soft_cap)
+        return logits

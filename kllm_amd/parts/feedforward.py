@@ -94,7 +94,8 @@ class GatedFeedForward(Part):
             normed = linear_into(ctx, h, self.w_down, sink, "ffn.down", w_tiled=self._tiled.get("down"))
             if normed is not None:
                 return normed
-        return linear(ctx, h, self.w_down, "ffn.down")
+            return linear(ctx, h, self.w_down, "ffn.down")
+        return decode_linear(ctx, h, self.w_down, "ffn.down", self._tiled.get("down"))
 
 
 @register_part("feed_forward", "dense_mlp")

@@ -72,6 +72,17 @@ class RMSNorm(Part):
         return x
 
 
+def pending_sums(delta):
+    """What a norm is to add to the stream first, as arguments of ``K.group_norm_add``."""
+    if delta is None:
+        return {}
+    if isinstance(delta, Normed):
+        raise ValueError("a residual product cannot stand for this norm")
+    if isinstance(delta, ScaledSum):
+        return {"deltas": delta.deltas, "bias": delta.bias, "mult": delta.mult}
+    return {"deltas": [delta]}
+
+
 @register_part("norm", "group_rmsnorm")
 class GroupRMSNorm(Part):
     """RMS norm in groups: the channels are cut into ``groups`` equal consecutive parts, each
@@ -98,24 +109,49 @@ class GroupRMSNorm(Part):
     def bind(self, weights):
         self.weight = weights[self.tensor_name("weight")]
 
-    @staticmethod
-    def _sum(delta):
-        if delta is None:
-            return {}
-        if isinstance(delta, Normed):
-            raise ValueError("group_rmsnorm: a residual product cannot stand for this norm")
-        if isinstance(delta, ScaledSum):
-            return {"deltas": delta.deltas, "bias": delta.bias, "mult": delta.mult}
-        return {"deltas": [delta]}
-
     def forward(self, ctx, x, delta=None, rows=None, tag="xn", normed_ok=False):
         n = rows.numel() if rows is not None else x.shape[0]
         out = ctx.buf(tag, (n, self.size), self.runtime.dtype)
         K.group_norm_add(x, weight=self.weight, out=out, rows=rows, groups=self.groups, eps=self.eps,
-                         **self._sum(delta))
+                         **pending_sums(delta))
         return out
 
     def add(self, ctx, x, delta):
         if delta is not None:
-            K.group_norm_add(x, **self._sum(delta))
+            K.group_norm_add(x, **pending_sums(delta))
+        return x
+
+
+@register_part("norm", "layernorm")
+class LayerNorm(Part):
+    """Layer norm: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b over the channels, in 32-bit.  It
+    also adds what is pending to the residual stream: a plain delta, or a ``ScaledSum`` of
+    sub-layers that ran side by side.
+
+    Parameters: ``size``, ``eps``.  Tensors: ``<prefix>.weight`` [size], ``<prefix>.bias`` [size]."""
+    graph_safe = True
+    records_launches = True
+
+    def __init__(self, spec, runtime):
+        super().__init__(spec, runtime)
+        self.size = int(self.param("size"))
+        self.eps = float(self.param("eps"))
+        self.weight = self.bias = None
+
+    def weight_specs(self):
+        return [WeightSpec(self.tensor_name("weight"), (self.size,), "vector"),
+                WeightSpec(self.tensor_name("bias"), (self.size,), "vector")]
+
+    def bind(self, weights):
+        self.weight, self.bias = weights[self.tensor_name("weight")], weights[self.tensor_name("bias")]
+
+    def forward(self, ctx, x, delta=None, rows=None, tag="xn", normed_ok=False):
+        n = rows.numel() if rows is not None else x.shape[0]
+        out = ctx.buf(tag, (n, self.size), self.runtime.dtype)
+        K.group_norm_add(x, weight=self.weight, norm_bias=self.bias, out=out, rows=rows, eps=self.eps, **pending_sums(delta))
+        return out
+
+    def add(self, ctx, x, delta):
+        if delta is not None:
+            K.group_norm_add(x, **pending_sums(delta))
         return x

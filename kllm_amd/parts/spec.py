@@ -10,7 +10,7 @@ that an earlier run wrote instead of writing one.
 
 from __future__ import annotations
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from typing import Any, Dict, List, Optional, Tuple
 
 
@@ -63,6 +63,15 @@ class CacheNeed:
                     self.keep_first if self.window else 0)
         return ("state", self.dtype) + tuple(self.state_shape)
 
+    def alike(self, other: "CacheNeed") -> bool:
+        """Whether what is kept has the same form, whatever the windows."""
+        return replace(self, window=0, keep_first=0).group_key() == replace(other, window=0, keep_first=0).group_key()
+
+    def covering(self, other: "CacheNeed") -> "CacheNeed":
+        """This need with a window wide enough for a reader with ``other`` too (see ``alike``)."""
+        window = max(self.window, other.window) if self.window and other.window else 0
+        return replace(self, window=window, keep_first=max(self.keep_first, other.keep_first) if window else 0)
+
 
 class PartSpec:
     """A registered part kind plus its parameters.  ``prefix`` is the start of
@@ -100,7 +109,8 @@ class LayerSpec:
 class Run:
     """One entry of the running order: run ``layer``; ``cache_of`` is None for
     a cache of its own, or the index of an earlier entry of the schedule whose
-    cache this run reads (it then writes none).  ``add``: which of the model's step vectors is
+    cache this run reads (it then writes none; the cache is kept for the wider of
+    the two windows).  ``add``: which of the model's step vectors is
     added to the stream in front of this run (None: none)."""
     layer: int
     cache_of: Optional[int] = None
