@@ -28,6 +28,9 @@ Other workloads, each printing one JSON line of its own (``--model`` chooses the
     --workload puladra         prefill and decode of a Puladra model (windowed attention behind short convolutions beside
                                retention, in turn with gated linear attention; experts without gates, an input by the
                                token, layers that run twice) beside Lugetar, Natenex and Llama
+    --workload bevadra         prefill and decode of a Bevadra model (latent attention behind a window in turn with windowed
+                               attention with a sink, a distance bias and an output gate, every second one reading
+                               an earlier layer's keys and values; parallel layers) beside Natenex, Nusilix and Llama
     --workload nusilix         prefill and decode of a Nusilix model (every fourth layer recurrent)
                                beside a Llama model of the same layer sizes (--sizes NAME; all if
                                not given)
@@ -64,8 +67,8 @@ def main(argv=None):
     ap.add_argument("--model", default="tinyllama-1.1b", choices=["tinyllama-1.1b", "llama2-7b", "llama3-8b"],
                     help="whose sizes to run (the default is the headline configuration)")
     ap.add_argument("--extra", default="", help="engine options for experiments: key=value,key=value (ints or words)")
-    ap.add_argument("--workload", default="headline", choices=["headline", "decode-run", "prefill-chunks", "mixed", "nusilix", "ribovik", "natenex", "lugetar", "puladra"])
-    ap.add_argument("--sizes", default="", help="layer sizes of the nusilix, ribovik, natenex, lugetar and puladra workloads (see benchmark.NUSILIX_SIZES)")
+    ap.add_argument("--workload", default="headline", choices=["headline", "decode-run", "prefill-chunks", "mixed", "nusilix", "ribovik", "natenex", "lugetar", "puladra", "bevadra"])
+    ap.add_argument("--sizes", default="", help="layer sizes of the nusilix, ribovik, natenex, lugetar, puladra and bevadra workloads (see benchmark.NUSILIX_SIZES)")
     ap.add_argument("--chunk", type=int, default=512, help="tokens per prompt portion (prefill-chunks, mixed)")
     ap.add_argument("--requests", type=int, default=32, help="requests of the mixed workload")
     ap.add_argument("--new-tokens", type=int, default=64, help="tokens each request of the mixed workload generates")
@@ -100,7 +103,7 @@ def main(argv=None):
     for item in filter(None, args.extra.split(",")):
         key, _, val = item.partition("=")
         extra[key] = int(val) if val.lstrip("-").isdigit() else (val or True)
-    if args.workload in ("nusilix", "ribovik", "natenex", "lugetar", "puladra"):
+    if args.workload in ("nusilix", "ribovik", "natenex", "lugetar", "puladra", "bevadra"):
         names = [args.sizes] if args.sizes else sorted(B.NUSILIX_SIZES)
         res = {"workload": args.workload, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic",
                "weights": "random", "context": args.context}

@@ -442,6 +442,24 @@ def puladra_config(width, heads, kv_heads, head_dim, ff, layers, vocab, window=1
     return cfg
 
 
+# Bevadra beside Natenex, Nusilix and Llama: layers in turn latent attention (Natenex' sizes) and attention
+# (Llama's heads), both behind a window of half the context; every second attention layer reads the
+# keys and values of the one before it.  The feed-forward is gated and as wide as Llama's.
+def bevadra_config(width, heads, kv_heads, head_dim, ff, layers, vocab, window=1024) -> dict:
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": 3 * width // 4, "kv_rank": 512,
+              "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}, "mask": {"size": window}}
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+                 "mask": {"size": window}}
+    entries = []
+    for i in range(layers):
+        mixer = dict(attention) if i % 2 else latent
+        if i % 4 == 3:
+            mixer["kv_from"] = i - 2
+        entries.append({"type": "attention" if i % 2 else "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Bevadra", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": entries}
+
+
 def spread_routing(eng: Engine, seed: int = 0) -> None:
     """Random weights as the engine draws them (all small, corrections all near 1) send every
     token to the same experts.  A router with large weights and no correction spreads the
@@ -463,9 +481,9 @@ def spread_routing(eng: Engine, seed: int = 0) -> None:
 def measure_design_pair(sizes: dict, dtype: str, batches=(1, 8), context: int = 2048, prompt: int = 2048,
                         steps: int = 64, delta_every: int = 4, design: str = "nusilix", design_sizes=None) -> dict:
     """Prefill and decode throughput of a model of ``design`` ("nusilix", "ribovik", "natenex",
-    "lugetar", "puladra") and of a Llama model of the same layer sizes (for Natenex a Nusilix model too,
-    for Lugetar a Natenex and a Ribovik model, for Puladra a Lugetar and a Natenex model: the nearest
-    in kind), one after the other on this GPU."""
+    "lugetar", "puladra", "bevadra") and of a Llama model of the same layer sizes (for Natenex a Nusilix
+    model too, for Lugetar a Natenex and a Ribovik model, for Puladra a Lugetar and a Natenex model, for
+    Bevadra a Natenex and a Nusilix model: the nearest in kind), one after the other on this GPU."""
     import gc
     out = {}
     models = []
@@ -482,6 +500,10 @@ def measure_design_pair(sizes: dict, dtype: str, batches=(1, 8), context: int = 
         first = puladra_config(**sizes, **(design_sizes or {}), window=max(64, context // 2))
         models.append(("lugetar", lugetar_config(**sizes, **(design_sizes or {}), chunk=max(64, context // 2))))
         models.append(("natenex", natenex_config(**sizes, window=max(64, context // 2))))
+    elif design == "bevadra":
+        first = bevadra_config(**sizes, window=max(64, context // 2))
+        models.append(("natenex", natenex_config(**sizes, window=max(64, context // 2))))
+        models.append(("nusilix", nusilix_config(delta_every=delta_every, **sizes)))
     else:
         first = nusilix_config(delta_every=delta_every, **sizes)
     for name, cfg in [(design, first)] + models + [("llama", llama_config(**sizes))]:

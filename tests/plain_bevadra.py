@@ -52,7 +52,9 @@ def window_of(m):
 
 
 def visible(n, window):
-    return torch.tensor([[sees(i, j, window) for j in range(n)] for i in range(n)])
+    """[n, n]: ``sees`` for every pair of positions."""
+    back = torch.arange(n)[:, None] - torch.arange(n)[None, :]
+    return (back >= 0) & (back < (window or n + 1))
 
 
 def rotate_halves(x, positions, rot):

@@ -1,0 +1,699 @@
+"""Bevadra on the GPU against the plain implementation (tests/plain_bevadra.py), in 32-bit and in
+bfloat16: each kernel alone (the norm around the mean, biases and padding in front of attention,
+learned sinks with a distance bias behind a window and a gate on the output, latents behind a
+window, a gate per head, the soft cap), each mixer alone, queries aimed at a key just inside and
+just outside a window, at page borders and hundreds of positions back, in prompts and while
+decoding, through a layer's own keys and through another layer's; then the engine through the trace
+replayer (whole prompts, decoding token by token, portions down to two tokens, mixed batches on few
+pages that are used again), configurations drawn from a seed, a batch against each of its requests
+alone, long decoding, and greedy generation through the scheduler and the command line."""
+
+import copy
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+import bevadra_tiny as T
+import plain_bevadra as P
+import traces
+
+pytestmark = pytest.mark.gpu
+
+DTYPES = ["float32", "bfloat16"]
+TD = {"float32": torch.float32, "bfloat16": torch.bfloat16}
+F64 = torch.float64
+# Logits: root mean square of the difference (mean taken off) over that of the plain model's logits.
+# A position's limit is five times what rounding of the products' inputs alone does to the plain
+# model there, where that is more (the engine also keeps queries, keys, values, probabilities and
+# latents in the compute type).
+TOL = {"float32": 3e-5, "bfloat16": 6e-2}
+WORST = {"float32": 0.0, "bfloat16": 0.0}
+# Aimed scores of 30 and values far larger than the others magnify the rounding of queries and
+# keys in bfloat16; a key that is wrongly seen or not seen moves the aimed rows by 0.3 and more
+# (checked in each test).
+AIMED_TOL = {"float32": 6e-5, "bfloat16": 0.12}
+NOISE = {"float32": 2.0 ** -22, "bfloat16": 2.0 ** -8}
+
+
+def rel(got, want):
+    got, want = torch.as_tensor(got, dtype=F64), torch.as_tensor(want, dtype=F64)
+    return float((got - want).norm() / want.norm().clamp_min(1e-30))
+
+
+def i32(x):
+    return torch.tensor(x, dtype=torch.int32, device="cuda")
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    made = {}
+
+    def get(name, seed=13, weights=None, tag=""):
+        key = (name, seed, tag)
+        if key not in made:
+            d = tmp_path_factory.mktemp(f"bevadra_{name}_{seed}_{tag}")
+            made[key] = T.write_model(str(d), T.CONFIGS[name], seed=seed, weights=weights)
+        return made[key]
+    return get
+
+
+def make_requests(cfg, lengths, seed):
+    return {f"r{i}": T.tokens(cfg, n, seed * 100 + i) for i, n in enumerate(lengths)}
+
+
+def row_error(got, want):
+    d, w = got - want, want - want.mean()
+    return float(np.sqrt(((d - d.mean()) ** 2).mean()) / np.sqrt((w ** 2).mean()))
+
+
+class Expected(dict):
+    """{request: logits of the plain model}; ``slack``: how far the plain model's own rows move when
+    the inputs of its products are rounded."""
+    slack = None
+
+
+def expected(model_dir, cfg, requests, dtype):
+    w = T.read_weights(model_dir, as_stored_in=dtype)
+    out = Expected({rid: P.forward(cfg, w, toks).numpy() for rid, toks in requests.items()})
+    g = torch.Generator().manual_seed(1)
+
+    def noisy(t):
+        return t * (1.0 + NOISE[dtype] * (2.0 * torch.rand(t.shape, generator=g, dtype=F64) - 1.0))
+    out.slack = {}
+    for rid, toks in requests.items():
+        moved = [P.forward(cfg, w, toks, rounded=noisy).numpy() for _ in range(2)]
+        out.slack[rid] = [max(row_error(m[p], out[rid][p]) for m in moved) for p in range(len(toks))]
+    return out
+
+
+def replay(model_dir, dtype, steps, max_tokens, slots=4, **opts):
+    from kllm_amd.engine import EngineOptions
+    from kllm_amd.replay import Replayer
+    options = EngineOptions(dtype=dtype, max_tokens=max_tokens, max_model_len=1 << 30, max_requests=slots,
+                            poison_freed_pages=True, **opts)
+    rep = Replayer(model_dir, dtype, max_tokens, options=options)
+    outs = [rep.step(s["entries"], s["end"]) for s in steps]
+    assert not rep.engine.cache.requests
+    rep.engine.cache.check_invariants()
+    assert all(p.free_pages == p.num_pages for p in rep.engine.cache.pools)
+    return traces.collect(steps, outs), rep
+
+
+def compare(rows, want, dtype, requests, tol=None):
+    """Every position within its limit in float32.  In bfloat16 one position in fifty (or one) may lie
+    over its limit, none over twice it; and four positions in five are within the limit without the
+    estimate of rounding."""
+    worst, over, count, leaning = 0.0, [], 0, 0
+    for rid, toks in requests.items():
+        for p in range(len(toks)):
+            got = rows[(rid, p)].astype(np.float64)
+            assert np.isfinite(got).all(), (rid, p)
+            err = row_error(got, want[rid][p])
+            limit = max(tol or TOL[dtype], 5.0 * want.slack[rid][p])
+            count += 1
+            leaning += err >= (tol or TOL[dtype])
+            if dtype == "bfloat16" and limit <= err < 2.0 * limit:
+                over.append((rid, p, err, limit))
+                continue
+            worst = max(worst, err * TOL[dtype] / limit)
+            assert err < limit, f"{rid} position {p}: off by {err} (limit {limit})"
+    assert len(rows) == sum(len(t) for t in requests.values())
+    assert len(over) <= max(1, count // 50), over
+    assert leaning <= max(3, count // 5), (leaning, count)
+    WORST[dtype] = max(WORST[dtype], worst)
+    return worst
+
+
+# ----------------------------------------------------------------------------- small kernels
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d", [3, 50, 64, 260, 1000, 2048, 4100, 9001])
+def test_norm_around_the_mean_with_what_is_pending(d, dtype):
+    """Two sums in slices and a bias go into the stream, the row is normed around its mean; then chosen
+    rows alone, and the addition alone."""
+    from kllm_amd import kernels as K
+    g = torch.Generator().manual_seed(d)
+    n, eps = 7, 1e-4
+    x = 5.0 + torch.randn(n, d, generator=g)
+    a, b = torch.randn(3, n, d, generator=g), torch.randn(n, d, generator=g)
+    bias, w, wb = (torch.randn(d, generator=g) for _ in range(3))
+    want_x = x.double() + 0.5 * (a.double().sum(0) + b.double() + bias.double())
+    want = P.layer_norm(want_x, w.double(), wb.double(), eps)
+    xd, out = x.cuda(), torch.empty(n, d, device="cuda", dtype=TD[dtype])
+    K.group_norm_add(xd, [a.cuda(), b.cuda()], bias=bias.cuda(), mult=0.5, weight=w.cuda(), norm_bias=wb.cuda(), out=out, eps=eps)
+    tol = 3e-6 if dtype == "float32" else 5e-3
+    assert rel(xd.cpu(), want_x) < 1e-6 and rel(out.float().cpu(), want) < tol
+    rows = i32([4, 0, 4])
+    out = torch.empty(3, d, device="cuda", dtype=TD[dtype])
+    K.group_norm_add(xd, weight=w.cuda(), norm_bias=wb.cuda(), out=out, rows=rows, eps=eps)
+    assert rel(out.float().cpu(), want[[4, 0, 4]]) < tol
+    without = torch.empty(3, d, device="cuda", dtype=TD[dtype])
+    K.group_norm_add(xd, weight=w.cuda(), out=without, rows=rows, eps=eps)
+    assert rel(without.float().cpu(), out.float().cpu()) > 0.1            # an RMS norm is another one
+
+
+def test_soft_cap_on_logits():
+    from kllm_amd import kernels as K
+    z = 40.0 * torch.randn(5, 777, generator=torch.Generator().manual_seed(0))
+    x = z.cuda()
+    K.soft_cap(x, 12.5)
+    assert (x.cpu().double() - P.soft_cap(z.double(), 12.5)).abs().max() < 1e-5
+    assert float(x.abs().max()) <= 12.5
+
+
+class Pages:
+    """A hand-made pool: requests' pages in a shuffled order, everything not written is NaN."""
+
+    def __init__(self, lengths, elems, page, dtype, seed):
+        g = torch.Generator().manual_seed(seed)
+        self.need = [-(-n // page) for n in lengths]
+        order = torch.randperm(sum(self.need) + 2, generator=g).tolist()
+        table = torch.full((len(lengths), max(self.need)), -1, dtype=torch.int32)
+        for s, c in enumerate(self.need):
+            for j in range(c):
+                table[s, j] = order.pop()
+        self.host, self.table, self.page = table, table.cuda(), page
+        self.pages = torch.full((sum(self.need) + 2, elems), float("nan"), device="cuda", dtype=dtype)
+
+    def with_holes(self, lows):
+        """(pages, table) in which request s's pages wholly in front of position lows[s] are gone: NaN,
+        and -1 in the table."""
+        pages, table = self.pages.clone(), self.host.clone()
+        for s, low in enumerate(lows):
+            for j in range(min(low // self.page, self.need[s])):
+                pages[table[s, j]] = float("nan")
+                table[s, j] = -1
+        return pages, table.cuda()
+
+
+ATTENTION_CASES = [  # H, KV, dk, dv, window
+    (4, 2, 24, 40, 20), (4, 1, 64, 64, 48), (6, 2, 64, 32, 100), (2, 1, 128, 128, 0), (5, 5, 10, 14, 7), (8, 2, 96, 96, 1),
+    (20, 1, 32, 32, 33), (3, 3, 200, 160, 17), (34, 2, 48, 64, 130)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,KV,dk,dv,window", ATTENTION_CASES)
+def test_biases_sinks_slopes_window_and_gate_in_the_attention_kernels(H, KV, dk, dv, window, dtype):
+    """Sums of the projections (two slices of a wider product) through the append with biases and
+    padding, in portions; then every attention kernel against a plain softmax with a sink: the one
+    that takes every size, single tokens in 1, 4 and 8 slices, prompts in blocks by every choice of
+    kernel, whole and in portions that start in the middle, pages behind the window gone.  Queries are
+    aimed at keys at the window's edges."""
+    from kllm_amd import kernels as K
+    dt, page, G = TD[dtype], 16, H // KV
+    width = next(v for v in K.PREFILL_HEAD_DIMS if v >= max(dk, dv))
+    g = torch.Generator().manual_seed(H * 100 + dk + window)
+    lengths = [291, 37]
+    n, scale = sum(lengths), 1.1 * dk ** -0.5
+    C, off = (H + KV) * dk + KV * dv, 3
+    raw = torch.randn(n, off + C + H * dv, generator=g)
+    bias, sinks = 0.3 * torch.randn(C, generator=g), 0.5 + 1.5 * torch.randn(H, generator=g)
+    i_in, i_out = 270, 280
+    W = window or 10 ** 6
+    pairs = [(i_in, max(i_in - W + 1, 0)), (i_out, i_out - W)] if i_out >= W else [(i_in, 3)]
+    for i, j in pairs:                      # query i and key j long and alike (their biases taken off)
+        u = torch.randn(dk, generator=g)
+        u = u / u.norm() * (28.0 / scale) ** 0.5
+        raw[i, off:off + H * dk] = u.repeat(H) - bias[:H * dk]
+        raw[j, off + H * dk:off + (H + KV) * dk] = u.repeat(KV) - bias[H * dk:(H + KV) * dk]
+    b = raw[:, off:off + C].double() + bias.double()
+    q, k, v = b[:, :H * dk].reshape(n, H, dk), b[:, H * dk:(H + KV) * dk].reshape(n, KV, dk), b[:, (H + KV) * dk:].reshape(n, KV, dv)
+    if dtype == "bfloat16":                 # what the kernels read is what was stored
+        q, k, v = (t.to(torch.bfloat16).double() for t in (q, k, v))
+    cut = lengths[0]
+    # rows of the aimed scores change far more than the others, so the rows are compared one by one
+    want = torch.cat([P.attend(q[a:e], k[a:e], v[a:e], scale, window, sinks.double()) for a, e in ((0, cut), (cut, n))])
+    gates = torch.sigmoid(raw[:, off + C:].double()).reshape(n, H, dv)
+    wanted = torch.zeros(n, H, width, dtype=F64)
+    wanted[..., :dv] = want * gates
+    cache = Pages(lengths, 2 * KV * page * width, page, dt, dk)
+    sums = torch.stack([raw * 0.25, raw * 0.75]).cuda()
+    qs = torch.empty(n, H * width, device="cuda", dtype=dt)
+    place = lambda pages: pages.view(-1, 2, KV, page * width)
+    cuts = [[0, 150, 289, 291], [0, 0, 20, 37]]
+    for step in range(3):
+        spans = [(s, cuts[s][step], cuts[s][step + 1]) for s in range(2) if cuts[s][step + 1] > cuts[s][step]]
+        rows = torch.cat([torch.arange(a, e) + s * cut for s, a, e in spans])
+        starts = [0]
+        for _, a, e in spans:
+            starts.append(starts[-1] + e - a)
+        part = sums[:, rows.cuda()].contiguous()
+        out = torch.empty(len(rows), H * width, device="cuda", dtype=dt)
+        single = all(e - a == 1 for _, a, e in spans)
+        args = (i32([p for _, a, e in spans for p in range(a, e)]), i32([j for j, (_, a, e) in enumerate(spans) for _ in range(a, e)]),
+                i32(list(range(len(spans)))), i32(starts), i32([a for _, a, _ in spans]))
+        table = cache.table[[s for s, _, _ in spans]].contiguous()
+        K.qkv_conv_append(K.Columns(part, off, C), None, 1, None, 0, single, out, place(cache.pages), *args, table, page, H, KV,
+                          dk, dv, width, bias=bias.cuda())
+        qs[rows.cuda()] = out
+        # without a cache: the same queries, nothing else
+        alone = torch.empty_like(out)
+        K.qkv_conv_append(K.Columns(part, off, H * dk), None, 1, None, 0, single, alone, None, *args, table, page, H, 0,
+                          dk, dv, width, bias=bias[:H * dk].contiguous().cuda())
+        assert torch.equal(alone, out)
+    assert rel(qs.float().cpu().reshape(n, H, width)[..., :dk], b[:, :H * dk].reshape(n, H, dk)) < (1e-6 if dtype == "float32" else 5e-3)
+    assert not qs.float().cpu().reshape(n, H, width)[..., dk:].any()
+    positions, span_of = i32(list(range(cut)) + list(range(lengths[1]))), i32([0] * cut + [1] * lengths[1])
+    slopes = torch.tensor(P.slopes(H), dtype=torch.float32, device="cuda")
+    opts = dict(slopes=slopes, sink=sinks.cuda(), gate=K.Columns(sums, off + C, H * dv))
+    pages, tol = place(cache.pages), 2e-5 if dtype == "float32" else 2e-2
+
+    def check(out, what, rows=None):
+        got, w = out.float().cpu().reshape(-1, H, width), wanted if rows is None else wanted[rows]
+        assert torch.isfinite(got).all() and rel(got, w) < tol, (what, rel(got, w))
+        for r in range(len(w)):
+            # (single rows of small gates and values: a little more)
+            assert rel(got[r], w[r]) < 3 * tol, (what, r, rel(got[r], w[r]))
+
+    args = (positions, span_of, cache.table, page, H, KV, width, window, scale)
+    out = torch.zeros(n, H * width, device="cuda", dtype=dt)
+    K.attn_generic(qs, out, pages, *args, **opts)
+    check(out, "generic")
+    # each option matters
+    aimed = [i for i, _ in pairs]
+    for change in ({"sink": None}, {"gate": None}) + (({"slopes": None},) if window != 1 else ()):
+        other = torch.zeros_like(out)
+        K.attn_generic(qs, other, pages, *args, **{**opts, **change})
+        assert rel(other.float().cpu().reshape(n, H, width), wanted) > 0.02, change
+    if window:
+        for wrong in (window - 1, window + 1):
+            if wrong:
+                other = torch.zeros_like(out)
+                K.attn_generic(qs, other, pages, *args[:7], wrong, scale, **opts)
+                assert max(rel(other.float().cpu().reshape(n, H, width)[i], wanted[i]) for i in aimed) > 0.2, wrong
+    for nslices in (1, 4, 8):
+        out = torch.zeros(n, H * width, device="cuda", dtype=dt)
+        part = torch.full((n * H * nslices * (width + 2),), float("nan"), device="cuda")
+        K.attn_decode(qs, out, part, pages, *args, nslices, **opts)
+        check(out, f"decode kernel, {nslices} slices")
+    last = [lengths[0] - 8, lengths[1] - 8]
+    lows = [max(p - W + 1, 0) for p in last]
+    holes, hole_table = cache.with_holes(lows)
+    rows = list(range(last[0], cut)) + list(range(cut + last[1], n))
+    for nslices in (1, 4):
+        out = torch.zeros(n, H * width, device="cuda", dtype=dt)
+        K.attn_decode(qs, out, part, place(holes), positions, span_of, hole_table, page, H, KV, width, window, scale, nslices,
+                      i32(rows), len(rows), **opts)
+        check(out[rows], f"decode kernel, pages gone, {nslices} slices", rows)
+    for firsts, pool, table in (([0, 0], pages, cache.table), ([141, 9], pages, cache.table), (last, place(holes), hole_table)):
+        lens = [lengths[s] - firsts[s] for s in range(2)]
+        rows = list(range(firsts[0], cut)) + list(range(cut + firsts[1], n))
+        qp = qs[rows].contiguous()
+        gate = K.Columns(sums[:, rows].contiguous(), off + C, H * dv)
+        m = len(rows)
+        tiles = [[t, 0] for t in range(0, lens[0], K.PREFILL_QUERY_BLOCK)] + [[t, 1] for t in range(lens[0], m, K.PREFILL_QUERY_BLOCK)]
+        for total, longest in ((0, 0), (10 ** 9, 10 ** 6), (1, 1)):          # every choice of the prompt kernel
+            out = torch.zeros(m, H * width, device="cuda", dtype=dt)
+            K.attn_prefill(qp, out, pool, i32(tiles), len(tiles), i32([0, lens[0], m]), i32(firsts), table, page, H, KV, width,
+                           window, scale, total, longest, slopes=slopes, sink=sinks.cuda(), gate=gate)
+            check(out, f"prompt kernel from {firsts}, keys {total}/{longest}", rows)
+
+
+LATENT_CASES = [(3, 40, 8, 20), (6, 160, 32, 70), (3, 448, 64, 33), (20, 96, 32, 1), (34, 128, 16, 130), (2, 512, 64, 2), (5, 14, 6, 9),
+                (4, 16, 8, 64)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,rank,dr,window", LATENT_CASES)
+def test_latents_behind_a_window(H, rank, dr, window, dtype):
+    """Folded queries over rows appended by the framework's own kernel, those of a token's window only
+    (in a second pass what lies behind it is gone: NaN pages and -1 in the table); a query looks along
+    the key at the window's oldest place and one along the key just behind it."""
+    from kllm_amd import kernels as K
+    dt, page, row, eps = TD[dtype], 16, rank + dr, 1e-5
+    g = torch.Generator().manual_seed(H * 1000 + rank)
+    lengths = [331, 19]
+    n, cut, scale = sum(lengths), lengths[0], 1.2 / row ** 0.5
+    cache = Pages(lengths, page * (row + rank), page, dt, rank)
+    sums = torch.randn(2, n, row + 5, generator=g)
+    weight = 1.0 + 0.2 * torch.randn(rank, generator=g)
+    pos = list(range(cut)) + list(range(lengths[1]))
+    span_of = [0] * cut + [1] * lengths[1]
+    rot = {"dims": dr, "base": 700.0}
+    raw = sums.double().sum(0)[:, 5:]
+    rows = torch.cat([P.rms_norm(raw[:, :rank], weight.double(), eps),
+                      torch.cat([P.rotate_halves(raw[a:a + 1, None, rank:], [pos[a]], rot)[:, 0] for a in range(n)])], dim=1)
+    q = torch.randn(n, H, row, generator=g)
+    i_in, i_out = 300, 320
+    for i, j in ((i_in, i_in - window + 1), (i_out, i_out - window)):
+        u = rows[j, :rank].float()
+        q[i, :, :rank] = u / u.norm() ** 2 * 25.0 / scale
+    freq = torch.tensor([700.0 ** (-2.0 * i / dr) for i in range(dr // 2)], dtype=F64)
+    cos, sin = torch.empty(n, dr // 2, device="cuda"), torch.empty(n, dr // 2, device="cuda")
+    K.rope_tables_freq(cos, sin, i32(pos), freq.cuda(), 1.0)
+    K.latent_kv_append(sums.cuda(), 5, weight.cuda(), eps, cos, sin, cache.pages, i32(pos), i32(span_of), cache.table, page, rank, dr)
+    stored = rows.to(dt).double()
+    qd = q.reshape(n, H * row).to("cuda", dt)
+    qq = qd.cpu().double().reshape(n, H, row)
+
+    def plain(window):
+        want = torch.zeros(n, H, rank, dtype=F64)
+        for a, e in ((0, cut), (cut, n)):
+            mask = P.visible(e - a, window)
+            for h in range(H):
+                s = (qq[a:e, h] @ stored[a:e].T * scale).masked_fill(~mask, float("-inf"))
+                want[a:e, h] = torch.softmax(s, -1) @ stored[a:e, :rank]
+        return want
+    want = plain(window)
+    assert rel(plain(window + 1)[i_out], want[i_out]) > 0.3 and (window == 1 or rel(plain(window - 1)[i_in], want[i_in]) > 0.3)
+    tol = 2e-5 if dtype == "float32" else 1.5e-2
+    low = [max(lengths[s] - 8 - window + 1, 0) for s in range(2)]
+    holes, hole_table = cache.with_holes(low)
+    tail = list(range(cut - 8, cut)) + list(range(n - 8, n))
+    for plain_kernel, slices in ((True, 1), (False, 1), (False, 4), (False, 32), (False, 0)):      # 0: four tokens a workgroup
+        out = torch.zeros(n, H * rank, device="cuda", dtype=dt)
+        part = torch.full((n * H * slices * (rank + 2),), float("nan"), device="cuda") if slices > 1 else None
+        K.attn_latent(qd, out, cache.pages, i32(pos), i32(span_of), cache.table, page, H, row, rank, scale, plain=plain_kernel,
+                      part=part, nslices=slices, window=window)
+        got = out.float().cpu().reshape(n, H, rank)
+        assert torch.isfinite(got).all() and rel(got, want) < tol, (plain_kernel, slices)
+        for i in range(n):
+            assert rel(got[i], want[i]) < 2 * tol, (plain_kernel, slices, i)
+        out = torch.zeros(len(tail), H * rank, device="cuda", dtype=dt)
+        K.attn_latent(qd[tail].contiguous(), out, holes, i32([pos[i] for i in tail]), i32([span_of[i] for i in tail]), hole_table,
+                      page, H, row, rank, scale, plain=plain_kernel, part=part, nslices=slices, window=window)
+        got = out.float().cpu().reshape(-1, H, rank)
+        assert torch.isfinite(got).all() and rel(got, want[tail]) < tol, (plain_kernel, slices, "pages gone")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("n,H,dv,rank", [(1, 3, 20, 40), (37, 6, 64, 160), (130, 5, 14, 14), (5, 20, 24, 96)])
+def test_a_gate_per_head_on_the_attended_latents(n, H, dv, rank, dtype):
+    from kllm_amd import kernels as K
+    g = torch.Generator().manual_seed(n + rank)
+    att = torch.randn(n, H * rank, generator=g).to(TD[dtype])
+    w_uv = (torch.randn(H * dv, rank, generator=g) / rank ** 0.5).to(TD[dtype])
+    gate = torch.randn(3, n, 7 + H, generator=g)
+    want = torch.einsum("nhr,hjr->nhj", att.double().reshape(n, H, rank), w_uv.double().reshape(H, dv, rank))
+    want = (want * torch.sigmoid(gate.double().sum(0)[:, 7:])[:, :, None]).reshape(n, H * dv)
+    out = torch.full((n, H * dv), float("nan"), device="cuda", dtype=TD[dtype])
+    K.latent_out(att.cuda(), w_uv.cuda(), out, H, dv, rank, gate=gate.cuda(), gate_column=7, gate_by_head=True)
+    assert rel(out.float().cpu(), want) < (2e-6 if dtype == "float32" else 8e-3)
+
+
+# ----------------------------------------------------------------------------- each mixer alone
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["A1", "L1", "R1"])
+def test_one_mixer_alone_whole_and_token_by_token(folders, name, dtype):
+    """A model of one mixer (R1: and one that reads its keys and values): the stream behind the layers
+    in one step, and the same from a prompt of 9 tokens followed by single tokens."""
+    from kllm_amd.engine import Engine, EngineOptions, StepEntry
+    cfg, d = T.CONFIGS[name], folders(name)
+    w = T.read_weights(d, as_stored_in=dtype)
+    toks = T.tokens(cfg, 70, 5)
+    want = []
+    P.forward(cfg, w, toks, taps=want)
+    eng = Engine.from_dir(d, EngineOptions(dtype=dtype, max_tokens=256, max_model_len=1 << 20, max_requests=2))
+    tol = 2e-6 if dtype == "float32" else 2e-2
+
+    def run(rid, portion):
+        taps = []
+        eng.step([StepEntry(rid, portion, [])], taps=taps)
+        return torch.stack([t.float().cpu() for t in taps[1:1 + len(want)]])
+    got = run("a", toks)
+    eng.release("a")
+    for i in range(len(want)):
+        assert rel(got[i], want[i]) < tol, i
+    got = torch.cat([run("b", toks[:9])] + [run("b", [t]) for t in toks[9:]], dim=1)
+    eng.release("b")
+    for i in range(len(want)):
+        for p in range(len(toks)):
+            assert rel(got[i][p], want[i][p]) < tol * 2, (i, p)
+
+
+# ----------------------------------------------------------------------------- aimed queries
+
+QUERY, KEY = 1, 2
+T.CONFIGS["W1"] = T._cfg(80, 64, 1e-5, 40.0, [T.attn(4, 2, 32, 20, window=24, ff=72), T.latent(2, 16, 8, 12, 20, 24, window=20)])
+T.CONFIGS["W2"] = T._cfg(96, 96, 1e-6, 40.0, [T.attn(4, 4, 64, window=40), T.attn(2, 1, 16, window=8, ff=40)])
+T.CONFIGS["W3"] = T._cfg(70, 80, 1e-5, 40.0, [T.attn(8, 2, 96, 128, window=130, ff=48)])
+# a reader whose window is wider than its source's, one whose window is narrower, one without a window
+T.CONFIGS["W4"] = T._cfg(80, 64, 1e-5, 40.0, [T.attn(4, 2, 32, 48, window=10, ff=40), T.attn(4, 2, 32, 48, window=37, source=0, ff=40)])
+T.CONFIGS["W5"] = T._cfg(80, 64, 1e-5, 40.0, [T.attn(4, 1, 64, window=70), T.latent(2, 8, 4, 8, 12, 16, window=5),
+                                               T.attn(4, 1, 64, window=19, source=0)])
+T.CONFIGS["W6"] = T._cfg(90, 72, 1e-5, 40.0, [T.latent(3, 24, 8, 20, 28, 44, window=29, ff=64), T.attn(2, 2, 16, window=16)])
+T.CONFIGS["W7"] = T._cfg(90, 96, 1e-5, 40.0, [T.latent(4, 64, 32, 64, 48, 208, window=100), T.latent(2, 8, 4, 8, 12, 20, ff=40)])
+T.CONFIGS["F1"] = T._cfg(90, 72, 1e-5, 40.0, [T.attn(8, 2, 32, window=0, ff=40)])
+T.CONFIGS["F2"] = T._cfg(90, 96, 1e-5, 40.0, [T.latent(3, 32, 16, 24, 40, 64, window=0)])
+T.CONFIGS["F3"] = T._cfg(90, 64, 1e-5, 40.0, [T.attn(8, 4, 24, window=12), T.attn(8, 4, 24, window=0, source=0, ff=48)])
+
+
+def aimed_prompt(cfg, n, seed, places):
+    """Random tokens other than the two aimed ones, with the key token and the query token put
+    at ``places`` ({position: token})."""
+    g = torch.Generator().manual_seed(seed)
+    toks = torch.randint(3, cfg["vocab"], (n,), generator=g).tolist()
+    for p, t in places.items():
+        toks[p] = t
+    return toks
+
+
+def check_aimed(folders, name, layer, dtype, reqs, shown):
+    """``shown``: (request, query position, key position, seen) for every aimed pair: the plain
+    model's row at the query must change a lot when a seen key's token is taken away, and when the
+    window is opened for a key that is not seen; then the engine's rows against the plain model's,
+    request whole, decoded at its end, and cut into portions."""
+    cfg = T.CONFIGS[name]
+    aim = T.aimed_latent if cfg["layers"][layer]["type"] == "latent_attention" else T.aimed_attention
+    # far keys: the score outweighs the distance bias of the heads with the smaller slopes
+    d = folders(name, weights=aim(cfg, P.random_weights(cfg, 21), QUERY, KEY, layer), tag="aimed")
+    want = expected(d, cfg, reqs, dtype)
+    w = T.read_weights(d, as_stored_in=dtype)
+    for rid, qpos, kpos, seen in shown:
+        if seen:
+            other = list(reqs[rid])
+            other[kpos] = 5
+            row = P.forward(cfg, w, other[:qpos + 1])[qpos].numpy()
+        elif kpos < qpos:
+            wider = copy.deepcopy(cfg)
+            wider["layers"][layer]["mixer"]["mask"]["size"] += 1
+            row = P.forward(wider, w, reqs[rid][:qpos + 1])[qpos].numpy()
+        else:
+            continue
+        assert rel(row, want[rid][qpos]) > 0.2, (rid, qpos, kpos, seen)
+    longest = max(len(t) for t in reqs.values())
+    for steps in (traces.whole(reqs), traces.bulk_then_tail(reqs, min(60, longest - 2)), traces.portions(reqs, seed=2)):
+        rows, _ = replay(d, dtype, steps, traces.peak_tokens(steps))
+        compare(rows, want, dtype, reqs, tol=AIMED_TOL[dtype])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,layer", [("W1", 0), ("W2", 0), ("W3", 0), ("W4", 1), ("W5", 2), ("W6", 0), ("W7", 0)])
+def test_a_query_aimed_at_the_edges_of_its_window(folders, name, layer, dtype):
+    cfg = T.CONFIGS[name]
+    W = cfg["layers"][layer]["mixer"]["mask"]["size"]
+    n = 2 * W + 25
+    qa = n - 3
+    reqs = {
+        "in": aimed_prompt(cfg, n, 1, {qa - W + 1: KEY, qa: QUERY}),        # the oldest position of the window
+        "out": aimed_prompt(cfg, n, 2, {qa - W: KEY, qa: QUERY}),           # one before it
+        "two": aimed_prompt(cfg, n, 3, {qa - W: KEY, qa: QUERY, qa - 1: QUERY}),    # the query before still sees it
+        "page": aimed_prompt(cfg, n, 4, {31: KEY, 31 + W - 1: QUERY}),      # the last slot of a page, just seen
+        "gone": aimed_prompt(cfg, n, 5, {31: KEY, 31 + W: QUERY}),
+        "next": aimed_prompt(cfg, n, 6, {32: KEY, 32 + W - 1: QUERY}),      # a page's first slot
+        "zero": aimed_prompt(cfg, n, 7, {0: KEY, W - 1: QUERY, W: QUERY}),
+        "short": aimed_prompt(cfg, W - 1, 8, {0: KEY, W - 2: QUERY}),       # shorter than the window: nothing masked
+        "ahead": aimed_prompt(cfg, 20, 9, {11: KEY, 10: QUERY}),
+    }
+    shown = [("in", qa, qa - W + 1, True), ("out", qa, qa - W, False), ("two", qa - 1, qa - W, True), ("page", 31 + W - 1, 31, True),
+             ("gone", 31 + W, 31, False), ("next", 32 + W - 1, 32, True), ("zero", W - 1, 0, True), ("zero", W, 0, False),
+             ("short", W - 2, 0, True), ("ahead", 10, 11, False)]
+    check_aimed(folders, name, layer, dtype, reqs, shown)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,layer", [("F1", 0), ("F2", 0), ("F3", 1)])
+def test_a_query_aimed_at_a_key_hundreds_of_positions_back(folders, name, layer, dtype):
+    """Where nothing is masked, also through the keys of a layer that itself reads a few positions."""
+    cfg = T.CONFIGS[name]
+    reqs = {
+        "far": aimed_prompt(cfg, 420, 1, {3: KEY, 410: QUERY}),
+        "first": aimed_prompt(cfg, 200, 2, {0: KEY, 190: QUERY}),
+        "page": aimed_prompt(cfg, 200, 3, {15: KEY, 171: QUERY}),             # the last slot of a page
+        "page2": aimed_prompt(cfg, 200, 3, {16: KEY, 171: QUERY}),            # the next page's first
+        "next": aimed_prompt(cfg, 40, 4, {30: KEY, 31: QUERY}),
+        "ahead": aimed_prompt(cfg, 40, 5, {31: KEY, 30: QUERY}),
+    }
+    shown = [("far", 410, 3, True), ("first", 190, 0, True), ("page", 171, 15, True), ("page2", 171, 16, True),
+             ("next", 31, 30, True), ("ahead", 30, 31, False)]
+    check_aimed(folders, name, layer, dtype, reqs, shown)
+
+
+# ----------------------------------------------------------------------------- the engine
+
+CASES = [("B1", [1, 5, 33, 130]), ("B2", [2, 17, 140]), ("B3", [3, 64, 65, 150]), ("B4", [90, 31, 4]), ("B5", [150, 49, 16, 17]),
+         ("B6", [210, 99, 7]), ("B7", [250, 3, 128])]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,lengths", CASES)
+def test_whole_prompts_decoding_portions_and_mixed_batches(folders, name, lengths, dtype):
+    """One configuration at a time through all four ways of cutting its requests into steps."""
+    cfg, d = T.CONFIGS[name], folders(name)
+    reqs = make_requests(cfg, lengths, 1)
+    want = expected(d, cfg, reqs, dtype)
+    steps = traces.whole(reqs)
+    rows, _ = replay(d, dtype, steps, traces.peak_tokens(steps))
+    compare(rows, want, dtype, reqs)
+    steps = traces.bulk_then_tail(reqs, 40)          # the tail crosses a window's and a page's border
+    rows, _ = replay(d, dtype, steps, traces.peak_tokens(steps))
+    compare(rows, want, dtype, reqs)
+    steps = traces.portions(reqs, seed=4)
+    assert min(len(s["entries"][0]["tokens"]) for s in steps if not s["end"]) == 2
+    rows, _ = replay(d, dtype, steps, traces.peak_tokens(steps))
+    compare(rows, want, dtype, reqs)
+    # more requests than may live at once, on so few pages and slots that they are used again
+    many = make_requests(cfg, lengths + [40, 7, 77, 12], 2)
+    want = expected(d, cfg, many, dtype)
+    steps, peak = traces.mixed(many, seed=5, max_live=4, tail=6, max_portion=20)
+    rows, _ = replay(d, dtype, steps, peak, slots=4)
+    compare(rows, want, dtype, many)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("seed", list(range(16)))
+def test_configurations_drawn_from_a_seed(folders, seed, dtype):
+    """Layer orders, sizes and constants that nobody chose: whole prompts and a mixed trace with
+    portions down to two tokens beside single tokens."""
+    name = f"X{seed}"
+    T.CONFIGS[name] = T.random_config(seed)
+    cfg, d = T.CONFIGS[name], folders(name, seed=seed + 100)
+    reqs = make_requests(cfg, [120, 3, 71, 18, 33], seed)
+    want = expected(d, cfg, reqs, dtype)
+    steps = traces.whole(reqs)
+    rows, _ = replay(d, dtype, steps, traces.peak_tokens(steps))
+    compare(rows, want, dtype, reqs)
+    steps, peak = traces.mixed(reqs, seed=seed, max_live=4, tail=9, max_portion=17)
+    rows, _ = replay(d, dtype, steps, peak)
+    compare(rows, want, dtype, reqs)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["B1", "B6"])
+def test_a_batch_against_each_request_alone(folders, name, dtype):
+    """The logits of a request do not depend on what else the step holds, beyond rounding: a
+    mixed trace against each of its requests replayed alone, cut the same way."""
+    cfg, d = T.CONFIGS[name], folders(name)
+    reqs = make_requests(cfg, [50, 23, 9, 71], 3)
+    steps, peak = traces.mixed(reqs, seed=1, max_live=3, tail=5, max_portion=16)
+    rows, _ = replay(d, dtype, steps, peak)
+    for rid in reqs:
+        alone = [{"step": i, "entries": [e for e in s["entries"] if e["id"] == rid],
+                  "end": [r for r in s["end"] if r == rid]} for i, s in enumerate(steps)]
+        alone = [s for s in alone if s["entries"]]
+        for i, s in enumerate(alone):
+            s["step"] = i
+        single, _ = replay(d, dtype, alone, peak)
+        for p in range(len(reqs[rid])):
+            assert rel(single[(rid, p)], rows[(rid, p)]) < (1e-5 if dtype == "float32" else 3e-2), (rid, p)
+
+
+def test_pages_that_are_given_back_hold_nothing_of_their_last_owner(folders):
+    """Few pages, seven requests one after another in pairs (freed pages are poisoned)."""
+    cfg, d = T.CONFIGS["B2"], folders("B2")
+    reqs = make_requests(cfg, [30, 45, 12, 64, 5, 33, 20], 6)
+    steps, peak = traces.mixed(reqs, seed=8, max_live=2, tail=3, max_portion=11)
+    rows, rep = replay(d, "float32", steps, peak, slots=2)
+    compare(rows, expected(d, cfg, reqs, "float32"), "float32", reqs)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["B1", "B5", "B6"])
+def test_long_decoding_over_page_and_window_borders(folders, name, dtype):
+    cfg, d = T.CONFIGS[name], folders(name)
+    reqs = make_requests(cfg, [260], 7)
+    steps = traces.bulk_then_tail(reqs, 257)
+    rows, rep = replay(d, dtype, steps, traces.peak_tokens(steps))
+    compare(rows, expected(d, cfg, reqs, dtype), dtype, reqs)
+    assert rep.engine.steps_repeated > 100                       # decode steps ran from their recorded commands
+
+
+@pytest.mark.parametrize("name", ["B2", "B6", "B7"])
+def test_the_kernel_for_every_size_and_the_matrix_core_kernels_agree(folders, name):
+    cfg, d = T.CONFIGS[name], folders(name)
+    reqs = make_requests(cfg, [300, 21, 150], 9)
+    steps, peak = traces.mixed(reqs, seed=2, max_live=3, tail=40, max_portion=70)
+    a, _ = replay(d, "bfloat16", steps, peak)
+    b, _ = replay(d, "bfloat16", steps, peak, attention="generic")
+    assert max(rel(a[k], b[k]) for k in a) < 3e-2
+    assert any(not np.array_equal(a[k], b[k]) for k in a)          # they are two kernels
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_recorded_steps_and_layers_change_no_bit(folders, dtype):
+    cfg, d = T.CONFIGS["B6"], folders("B6")
+    reqs = make_requests(cfg, [140, 21], 9)
+    steps, peak = traces.mixed(reqs, seed=2, max_live=2, tail=10, max_portion=12)
+    a, _ = replay(d, dtype, steps, peak)
+    c, _ = replay(d, dtype, steps, peak, extra={"no_repeated_layers": True, "no_repeated_steps": True, "launch_one_by_one": True})
+    assert all(np.array_equal(a[k], c[k]) for k in a)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["B1", "B2"])
+def test_greedy_generation_through_the_scheduler(folders, dtype, name):
+    from kllm_amd.engine import Engine, EngineOptions
+    cfg, d = T.CONFIGS[name], folders(name)
+    w = T.read_weights(d, as_stored_in=dtype)
+    prompts = [T.tokens(cfg, n, 40 + n) for n in (3, 11, 30, 6, 18)]
+    eng = Engine.from_dir(d, EngineOptions(dtype=dtype, max_tokens=1024, max_model_len=256, max_requests=4))
+    got = eng.generate(prompts, max_new_tokens=12, max_step_tokens=16, max_batch=3)
+    for prompt, ids in zip(prompts, got):
+        want = P.greedy(cfg, w, prompt, 12)
+        k = next((i for i, (a, b) in enumerate(zip(ids, want)) if a != b), 12)
+        if k < 12:      # a near tie may fall the other way; what was generated up to there agrees
+            assert dtype == "bfloat16", (ids, want)
+            lg = P.forward(cfg, w, prompt + want[:k])[-1]
+            top = torch.topk(lg, 2).values
+            assert float(top[0] - top[1]) < 0.2 * float(lg.std())
+    assert not eng.cache.requests
+
+
+def test_decode_steps_as_graphs_replayed_with_other_work_between(folders):
+    """Steps queued one ahead, ids on the device, recorded as HIP graphs and replayed many times with
+    eager steps of another request between the replays: the same ids as step by step."""
+    from kllm_amd.engine import Engine, EngineOptions
+    cfg, d = T.CONFIGS["B1"], folders("B1")
+    prompts = [T.tokens(cfg, n, 60 + n) for n in (7, 12, 5)]
+    eng = Engine.from_dir(d, EngineOptions(dtype="float32", max_tokens=2048, max_model_len=512, max_requests=4, graph_after_steps=1))
+    a = eng.generate(prompts, max_new_tokens=40, max_step_tokens=64, max_batch=3)
+    assert eng._graphs.captures > 0
+    plain = Engine.from_dir(d, EngineOptions(dtype="float32", max_tokens=2048, max_model_len=512, max_requests=4, graphs=False))
+    assert plain.generate(prompts, max_new_tokens=40, max_step_tokens=64, max_batch=3) == a
+    again = eng.generate(prompts[:1] + [T.tokens(cfg, 33, 5)] + prompts[1:], max_new_tokens=40, max_step_tokens=16, max_batch=3)
+    assert [again[0]] + again[2:] == a
+
+
+def test_the_command_line_programs_take_the_model(folders, tmp_path):
+    """bin/generate (greedy, float32) against the plain model's greedy continuation, and
+    bin/trace_run fed a trace on its standard input, one line a step."""
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    cfg, d = T.CONFIGS["B4"], folders("B4")
+    w = T.read_weights(d)
+    prompt = T.tokens(cfg, 9, 77)
+    p = subprocess.run([sys.executable, os.path.join(root, "bin", "generate"), "--model", d, "--dtype", "float32",
+                        "--ids", " ".join(map(str, prompt)), "--steps", "10"], capture_output=True, text=True, timeout=600)
+    assert p.returncode == 0, p.stderr[-2000:]
+    line = [l for l in p.stdout.splitlines() if l.startswith("generated:")][0]
+    assert [int(v) for v in line.split("[")[1].rstrip("]").split()] == P.greedy(cfg, w, prompt, 10)
+    reqs = make_requests(cfg, [37, 12], 8)
+    steps, peak = traces.mixed(reqs, seed=3, max_live=2, tail=4, max_portion=9)
+    out = tmp_path / "logits"
+    p = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", d, "--dtype", "float32",
+                        "--out", str(out), "--max-tokens", str(peak)], input="\n".join(json.dumps(s) for s in steps) + "\n",
+                       capture_output=True, text=True, timeout=600)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [l for l in p.stdout.splitlines() if l.startswith("done ")] == [f"done {s['step']}" for s in steps]
+    outs = [np.fromfile(out / f"{s['step']}.f32", dtype="<f4").reshape(-1, cfg["vocab"]) for s in steps]
+    compare(traces.collect(steps, outs), expected(d, cfg, reqs, "float32"), "float32", reqs)
+
+
+def test_zz_the_worst_difference_seen():
+    print("worst relative difference of logits:", WORST)
+    assert all(WORST[d] < TOL[d] for d in WORST)
