@@ -84,7 +84,9 @@ __global__ __launch_bounds__(kLatThreads) void latent_kv_append_kernel(
 }
 
 // out [n][r] = N(in row's r elements) * weight, the rows of `in` in_stride apart; one workgroup a row.
-template <typename T>
+// PER > 0: rows of up to PER * kLatThreads elements, which a thread keeps in registers, so that its
+// loads (a slice's all together) are one trip to memory each.
+template <typename T, int PER>
 __global__ __launch_bounds__(kLatThreads) void latent_norm_kernel(const float* __restrict__ in, int nsplit,
                                                                   long split_stride, long in_stride,
                                                                   const float* __restrict__ weight, float eps,
@@ -94,6 +96,25 @@ __global__ __launch_bounds__(kLatThreads) void latent_norm_kernel(const float* _
   const int tid = threadIdx.x;
   const float* src = in + t * in_stride;
   float ss = 0.f;
+  if constexpr (PER > 0) {
+    float v[PER], w[PER];
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      v[j] = 0.f;
+      w[j] = weight[min(tid + kLatThreads * j, r - 1)];
+    }
+    for (int s = 0; s < nsplit; ++s)
+#pragma unroll
+      for (int j = 0; j < PER; ++j) v[j] += src[s * split_stride + min(tid + kLatThreads * j, r - 1)];
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (tid + kLatThreads * j < r) ss = fmaf(v[j], v[j], ss);
+    const float rstd = 1.f / sqrtf(block_sum(ss, red) / (float)r + eps);
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      if (tid + kLatThreads * j < r) out[t * r + tid + kLatThreads * j] = from_f32<T>(v[j] * rstd * w[j]);
+    return;
+  }
   for (int i = tid; i < r; i += kLatThreads) {
     float v = 0.f;
     for (int s = 0; s < nsplit; ++s) v += src[s * split_stride + i];
@@ -223,7 +244,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     int max_pages, int page_size, unsigned page_magic, int H, int row, int rank, float scale, int window,
     float* __restrict__ part) {
   extern __shared__ float lat_red[];            // [kLatWaves - 1][NR * 4 + 2][64]
-  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int lane = threadIdx.x % kWave, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
   const int g = lane / 16, c = lane % 16;
   const int t = blockIdx.x, h0 = blockIdx.y * 16;
   const int head = min(h0 + c, H - 1);
@@ -251,9 +272,12 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
   // tokens and heads alone leave CUs idle) and, within a slice, to the waves.
   const int nslices = gridDim.z, slice = blockIdx.z;
   const int tiles = (len + 31) / 32;
+  const unsigned k_lane = c * row + 8 * g, v_lane = c * page_size + 4 * g;       // this lane's place in a half's rows and latents
   for (int tile = lo / 32 + slice * kLatWaves + wave; tile < tiles; tile += kLatWaves * nslices) {
     const int kb = tile * 32;
-    // a half (16 keys) lies in one page (pages hold a multiple of 16 slots)
+    // A half (16 keys) lies in one page (pages hold a multiple of 16 slots).  Loads carry no branch,
+    // so that many are in flight: a half that is not read takes page 0, whose rows make scores that
+    // are masked (a row is one key's alone) and whose latents are replaced by zeros.
     const bf16_t* pbase[2];
     int slot0[2];
     bool live[2];
@@ -262,29 +286,64 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
       const int k0 = kb + 16 * u;
       live[u] = k0 < len && k0 + 16 > lo;                    // (a half behind the window may lie in a page that is gone)
       const int pi = live[u] ? (int)(__umulhi((unsigned)k0, page_magic) >> 3) : 0;   // k0 / page_size (see the launch)
-      const int page = live[u] ? table[pi] : 0;
-      pbase[u] = cache + (long)page * page_elems;
+      // (the same in every lane: said so explicitly, which keeps the addresses on the scalar unit)
+      const int page = __builtin_amdgcn_readfirstlane(table[pi]);
+      pbase[u] = cache + (long)(live[u] ? page : 0) * page_elems;
       slot0[u] = live[u] ? k0 - pi * page_size : 0;
     }
-    floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
-    auto score_step = [&](int ks, const bf16x8& qb) {
-      const int d0 = 32 * ks + 8 * g;
-      const bool in = d0 < row;
-#pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        const bf16x8 a = (in && live[u]) ? *reinterpret_cast<const bf16x8*>(pbase[u] + (long)(slot0[u] + c) * row + d0) : zero8;
-        s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qb, s[u], 0, 0, 0);
-      }
+    const bf16_t* krow[2] = {pbase[0] + (long)slot0[0] * row, pbase[1] + (long)slot0[1] * row};      // + this lane's place
+    const bf16_t* vt[2] = {pbase[0] + (long)page_size * row + slot0[0], pbase[1] + (long)page_size * row + slot0[1]};
+    // ---- the latents' pieces, RB at a time: the first are asked for before the scores are worked on
+    constexpr int RB = 8;
+    struct Piece {
+      bf16x4 v[RB][2];
     };
-    if constexpr (KS > 0) {
+    auto v_fetch = [&](int r0) -> Piece {
+      Piece P;
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks)
-        if (ks < ksteps) score_step(ks, qreg[ks]);
+      for (int j = 0; j < RB; ++j)
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+          P.v[j][u] = *reinterpret_cast<const bf16x4*>(vt[u] + (long)(16 * min(r0 + j, nr - 1)) * page_size + v_lane);
+      return P;
+    };
+    floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
+    Piece piece;
+    if constexpr (KS > 0) {
+      constexpr int KB = KS % 6 == 0 ? 6 : KS % 5 == 0 ? 5 : 4;   // steps whose pieces of the keys are asked for together
+      static_assert(KS % KB == 0, "whole groups of steps");
+#pragma unroll
+      for (int k0 = 0; k0 < KS; k0 += KB) {
+        bf16x8 a[KB][2];
+#pragma unroll
+        for (int j = 0; j < KB; ++j)
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            const int d0 = 32 * (k0 + j) + 8 * g;
+            a[j][u] = *reinterpret_cast<const bf16x8*>(krow[u] + k_lane + (unsigned)(d0 < row ? 32 * (k0 + j) : 0));
+          }
+        if (k0 + KB >= KS) piece = v_fetch(0);
+        __builtin_amdgcn_sched_barrier(0);                   // (two groups in flight at most: registers)
+#pragma unroll
+        for (int j = 0; j < KB; ++j)
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            const bool in = 32 * (k0 + j) + 8 * g < row;     // beyond a row: another slot's, anything
+            s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(in ? a[j][u] : zero8, qreg[k0 + j], s[u], 0, 0, 0);
+          }
+      }
     } else {
       for (int ks = 0; ks < ksteps; ++ks) {
-        const int d0 = 32 * ks + 8 * g;
-        score_step(ks, (d0 < row && head_ok) ? *reinterpret_cast<const bf16x8*>(qrow + d0) : zero8);
+        const int d0 = 32 * ks + 8 * g, da = d0 < row ? d0 : 0;
+        const bf16x8 qv = *reinterpret_cast<const bf16x8*>(qrow + da);
+        const bf16x8 qb = (d0 < row && head_ok) ? qv : zero8;
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const bf16x8 a = *reinterpret_cast<const bf16x8*>(krow[u] + c * row + da);
+          s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(d0 < row ? a : zero8, qb, s[u], 0, 0, 0);
+        }
       }
+      piece = v_fetch(0);
     }
     // ---- online softmax for this lane's head over its 8 keys, then over the 4 lanes of the column
     float tmax = -INFINITY;
@@ -314,20 +373,25 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     l = l * alpha + psum;
     m = m_new;
     // ---- the weighted sum of the latents: slots beyond the last key may hold anything
-    const bf16_t* vt[2] = {pbase[0] + (long)page_size * row + slot0[0] + 4 * g,
-                           pbase[1] + (long)page_size * row + slot0[1] + 4 * g};
+    const bool edge = !live[0] || kb + 32 > len;
 #pragma unroll
-    for (int r = 0; r < NR; ++r) {
-      if (r < nr) {
-        acc[r] *= alpha;
-        bf16x8 a;
+    for (int r0 = 0; r0 < NR; r0 += RB) {
+      const Piece now = piece;
+      if (r0 + RB < NR) piece = v_fetch(r0 + RB);
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          const bf16x4 v = live[u] ? *reinterpret_cast<const bf16x4*>(vt[u] + (long)(16 * r + c) * page_size) : bf16x4{0, 0, 0, 0};
+      for (int j = 0; j < RB; ++j) {
+        const int r = r0 + j;
+        if (r < nr) {
+          acc[r] *= alpha;
+          bf16x8 a;
 #pragma unroll
-          for (int i = 0; i < 4; ++i) a[4 * u + i] = (kb + 16 * u + 4 * g + i < len) ? v[i] : (bf16_t)0.f;
+          for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+              a[4 * u + i] = (!edge || (live[u] && kb + 16 * u + 4 * g + i < len)) ? now.v[j][u][i] : (bf16_t)0.f;
+          acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, acc[r], 0, 0, 0);
         }
-        acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, acc[r], 0, 0, 0);
       }
     }
   }
@@ -455,70 +519,98 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
     const int group_lo = first_key(positions[t_first + first], window, 0);   // ... and its first the earliest (pages before it may be gone)
     const bool mine = token_ok && wave >= first && wave <= last;
     const int* table = block_table + (long)span * max_pages;
-    // ---- a tile's way into LDS: 16-byte pieces (a half, 16 keys, lies in one page).  For the built
-    // row sizes a thread's pieces of the NEXT tile are asked for before the products of this one
-    // and wait in registers meanwhile.
-    const int row8 = row / 8;
-    constexpr int KP = KS / 2, VP = NR / 4;     // pieces a thread: 32 rows x 4 KS / 256, 16 NR elements x 4 / 256
+    // ---- a tile's way into LDS, 16 bytes at a time.  Thread tid moves pieces tid % 8, + 8, ... of key row
+    // tid / 8, and 8 keys (part tid % 4) of elements tid / 4, + 64, ...: the same places in every tile.
+    // For the built row sizes the pieces of the NEXT tile are asked for before the products of this
+    // one and wait in registers meanwhile, their pages having been looked up a tile earlier, and no
+    // load has a branch around it: a half (16 keys, in one page) that nobody reads takes page 0;
+    // its scores are masked (a row is one key's alone), its latents replaced by zeros.
+    constexpr int KP = KS > 0 ? KS / 2 : 1, VP = NR / 4;      // pieces a thread: of 32 rows of up to 32 KS, of 16 NR elements
     struct Stage {
-      bf16x8 k[KP > 0 ? KP : 1], v[VP];
+      bf16x8 k[KP], v[VP];
     };
-    auto k_piece = [&](int i, int kb) -> bf16x8 {
-      const int kr = i / row8;                                // (for the built sizes: unrolled, i and row8 known per thread before the loop)
-      const int key = kb + kr;
-      if (i >= 32 * row8 || key >= group_len || key < group_lo) return zero8;
-      const int pi = page_index(key);
-      const long pg = table[pi];
-      return *reinterpret_cast<const bf16x8*>(cache + pg * page_elems + (long)(key - pi * page_size) * row + 8 * (i - kr * row8));
+    struct Halves {
+      int page[2];
     };
-    auto v_piece = [&](int i, int kb) -> bf16x8 {             // 8 keys of one element
-      const int e = i / 4, key = kb + 8 * (i % 4);
-      if (e >= rank || key >= group_len || key + 8 <= group_lo) return zero8;
-      const int pi = page_index(key);
-      const long pg = table[pi];
-      bf16x8 v = *reinterpret_cast<const bf16x8*>(cache + pg * page_elems + (long)page_size * row + (long)e * page_size +
-                                                  (key - pi * page_size));
-      if (key + 8 > group_len) {                              // slots behind the last key may hold anything
+    const int row8 = row / 8;
+    const int kr = tid / 8, kc = tid % 8, ve = tid / 4, vpart = tid % 4;
+    auto half_live = [&](int k0) { return k0 < group_len && k0 + 16 > group_lo; };
+    auto lookup = [&](int kb) -> Halves {
+      Halves P;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = key + j < group_len ? v[j] : (bf16_t)0.f;
+      for (int u = 0; u < 2; ++u) P.page[u] = table[half_live(kb + 16 * u) ? page_index(kb + 16 * u) : 0];
+      return P;
+    };
+    auto place = [&](const Halves& P, int k0, int u) -> const bf16_t* {      // the half's first row in its page
+      const bool live = half_live(k0);
+      return cache + (long)(live ? (u ? P.page[1] : P.page[0]) : 0) * page_elems;
+    };
+    auto slot_of = [&](int k0) { return half_live(k0) ? k0 - page_index(k0) * page_size : 0; };
+    auto k_load = [&](const bf16_t* rows, int m) -> bf16x8 {
+      const int piece = kc + 8 * m;
+      return *reinterpret_cast<const bf16x8*>(rows + 8 * (piece < row8 ? piece : 0));
+    };
+    auto v_load = [&](const bf16_t* cols, int m) -> bf16x8 {
+      return *reinterpret_cast<const bf16x8*>(cols + (long)min(ve + 64 * m, rank - 1) * page_size);
+    };
+    auto k_rows = [&](const Halves& P, int kb) {
+      const int u = kr / 16, k0 = kb + 16 * u;
+      return place(P, k0, u) + (long)(slot_of(k0) + kr % 16) * row;
+    };
+    auto v_cols = [&](const Halves& P, int kb) {
+      const int u = vpart / 2, k0 = kb + 16 * u;
+      return place(P, k0, u) + (long)page_size * row + slot_of(k0) + 8 * (vpart % 2);
+    };
+    auto k_store = [&](int m, const bf16x8& v) {
+      const int piece = kc + 8 * m;
+      if (piece < row8) *reinterpret_cast<bf16x8*>(ks + kr * KLD + 8 * piece) = v;
+    };
+    auto v_store = [&](int m, bf16x8 v, int kb) {
+      if (ve + 64 * m >= rank) return;
+      if (kb < group_lo || kb + 32 > group_len) {             // slots that may hold anything
+        const int key = kb + 8 * vpart;
+        const bool live = half_live(kb + 16 * (vpart / 2));
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = (live && key + j < group_len) ? v[j] : (bf16_t)0.f;
       }
-      return v;
-    };
-    auto k_store = [&](int i, const bf16x8& v) {
-      const int kr = i / row8;
-      if (i < 32 * row8) *reinterpret_cast<bf16x8*>(ks + kr * KLD + 8 * (i - kr * row8)) = v;
-    };
-    auto v_store = [&](int i, const bf16x8& v) {
-      if (i >= rank * 4) return;
-      bf16_t* dst = vs + (i / 4) * VLD + 8 * (i % 4);         // 8-byte aligned
+      bf16_t* dst = vs + (ve + 64 * m) * VLD + 8 * vpart;     // 8-byte aligned
       *reinterpret_cast<bf16x4*>(dst) = bf16x4{v[0], v[1], v[2], v[3]};
       *reinterpret_cast<bf16x4*>(dst + 4) = bf16x4{v[4], v[5], v[6], v[7]};
     };
-    auto fetch = [&](int kb) -> Stage {
+    auto fetch = [&](int kb, const Halves& P) -> Stage {
       Stage T;
+      const bf16_t *kp = k_rows(P, kb), *vp = v_cols(P, kb);
 #pragma unroll
-      for (int j = 0; j < KP; ++j) T.k[j] = k_piece(tid + 64 * kLatWaves * j, kb);
+      for (int m = 0; m < KP; ++m) T.k[m] = k_load(kp, m);
 #pragma unroll
-      for (int j = 0; j < VP; ++j) T.v[j] = v_piece(tid + 64 * kLatWaves * j, kb);
+      for (int m = 0; m < VP; ++m) T.v[m] = v_load(vp, m);
       return T;
     };
     Stage st;
+    Halves pages;
     const int kb0 = group_lo / 32 * 32;
-    if constexpr (KS > 0) st = fetch(kb0);
+    if constexpr (KS > 0) {
+      pages = lookup(kb0);
+      st = fetch(kb0, pages);
+      pages = lookup(kb0 + 32);
+    }
     for (int kb = kb0; kb < group_len; kb += 32) {
       __syncthreads();                                        // the tile before this one has been read
       if constexpr (KS > 0) {
 #pragma unroll
-        for (int j = 0; j < KP; ++j) k_store(tid + 64 * kLatWaves * j, st.k[j]);
+        for (int m = 0; m < KP; ++m) k_store(m, st.k[m]);
 #pragma unroll
-        for (int j = 0; j < VP; ++j) v_store(tid + 64 * kLatWaves * j, st.v[j]);
+        for (int m = 0; m < VP; ++m) v_store(m, st.v[m], kb);
       } else {
-        for (int i = tid; i < 32 * row8; i += 64 * kLatWaves) k_store(i, k_piece(i, kb));
-        for (int i = tid; i < rank * 4; i += 64 * kLatWaves) v_store(i, v_piece(i, kb));
+        pages = lookup(kb);
+        const bf16_t *kp = k_rows(pages, kb), *vp = v_cols(pages, kb);
+        for (int m = 0; 8 * m < row8; ++m) k_store(m, k_load(kp, m));
+        for (int m = 0; 64 * m < rank; ++m) v_store(m, v_load(vp, m), kb);
       }
       __syncthreads();
-      if constexpr (KS > 0) {
-        if (kb + 32 < group_len) st = fetch(kb + 32);         // (the same for all: no barrier inside)
+      if constexpr (KS > 0) {                                 // (beyond the last tile: a valid address, dropped)
+        st = fetch(kb + 32, pages);
+        pages = lookup(kb + 64);
       }
       if (!mine || kb >= len || kb + 32 <= lo) continue;
       // ---- scores
@@ -599,26 +691,35 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
   }
 }
 
-// The slices' results of one (token, head) become its output: weights exp(m_s - max m).
+// The slices' results of one (token, head) become its output: weights exp(m_s - max m).  A lane takes one
+// slice's maximum and sum (up to 64 slices) and works out its weight; the weights wait in LDS while
+// eight slices' outputs at a time are asked for.
 __global__ __launch_bounds__(kLatThreads) void attn_latent_merge_kernel(const float* __restrict__ part,
                                                                         bf16_t* __restrict__ out, int rank, int nslices) {
+  __shared__ float weight[kWave];
   const long th = blockIdx.x;
-  const float* rows = part + th * nslices * (rank + 2);
-  float M = -INFINITY;
-  for (int s = 0; s < nslices; ++s) M = fmaxf(M, rows[(long)s * (rank + 2) + rank]);
-  float l = 0.f;
-  for (int s = 0; s < nslices; ++s) {
-    const float ms = rows[(long)s * (rank + 2) + rank];
-    if (ms != -INFINITY) l += expf(ms - M) * rows[(long)s * (rank + 2) + rank + 1];
-  }
-  const float inv = 1.f / l;
+  const long stride = rank + 2;
+  const float* rows = part + th * nslices * stride;
+  const int lane = threadIdx.x % kWave;
+  const bool there = lane < nslices;
+  const float ms = there ? rows[lane * stride + rank] : -INFINITY;
+  const float ls = there ? rows[lane * stride + rank + 1] : 0.f;
+  const float M = wave_max(ms);                               // finite: some slice holds the token's own key
+  const float w = ms == -INFINITY ? 0.f : expf(ms - M);
+  const float inv = 1.f / wave_sum(w * ls);
+  if (threadIdx.x < kWave) weight[lane] = w * inv;            // 0 for a slice without a key
+  __syncthreads();
   for (int e = threadIdx.x; e < rank; e += kLatThreads) {
     float o = 0.f;
-    for (int s = 0; s < nslices; ++s) {
-      const float ms = rows[(long)s * (rank + 2) + rank];
-      if (ms != -INFINITY) o = fmaf(expf(ms - M), rows[(long)s * (rank + 2) + e], o);
+    for (int s0 = 0; s0 < nslices; s0 += 8) {
+      float v[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] = rows[min(s0 + j, nslices - 1) * stride + e];
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (s0 + j < nslices && weight[s0 + j] != 0.f) o = fmaf(weight[s0 + j], v[j], o);
     }
-    out[th * rank + e] = (bf16_t)(o * inv);
+    out[th * rank + e] = (bf16_t)o;
   }
 }
 
@@ -768,6 +869,120 @@ __global__ __launch_bounds__(kLatThreads) void latent_query_mfma_kernel(
   }
 }
 
+// The same two products for steps of many tokens, MFMA 32x32x16 (lane l: g = l/32, c = l%32: A[c][8g..],
+// B[8g..][c], D[8(i/4) + 4g + i%4][c]): a workgroup takes 64 tokens of a head, A = 32 outputs (rows of the
+// head's matrix), B = 32 tokens; a lane then holds pieces of four neighbouring outputs of one token.
+constexpr int kLatTokens = 64;
+
+// DS = d / 16.  The tokens' queries (their slices added, in the compute type) pass through LDS once
+// for all outputs; a wave takes every fourth piece of 32 outputs.
+template <int DS>
+__global__ __launch_bounds__(kLatThreads) void latent_query_block_kernel(
+    const float* __restrict__ q, int nsplit, long split_stride, const bf16_t* __restrict__ w_ukt,
+    const float* __restrict__ cos_t, const float* __restrict__ sin_t, bf16_t* __restrict__ out, int n, int H, int dr,
+    int rank) {
+  constexpr int d = 16 * DS, LD = d + 8;
+  __shared__ __attribute__((aligned(16))) bf16_t qs[kLatTokens * LD];
+  const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+  const int g = lane / 32, c = lane % 32;
+  const int h = blockIdx.x, t0 = blockIdx.y * kLatTokens;
+  const int hw = d + dr, half = dr / 2;
+  const long row_out = (long)H * (rank + dr);
+  for (int i = tid; i < kLatTokens * (d / 4); i += kLatThreads) {
+    const int tt = i / (d / 4), e = 4 * (i % (d / 4));
+    const float* in = q + ((long)min(t0 + tt, n - 1) * H + h) * hw + e;
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < nsplit; ++s)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] += in[s * split_stride + j];
+    *reinterpret_cast<bf16x4*>(qs + tt * LD + e) = bf16x4{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+  }
+  // the rotated part beside it
+  for (int i = tid; i < kLatTokens * half; i += kLatThreads) {
+    const int tt = i / half, e = i % half, t = t0 + tt;
+    if (t >= n) break;
+    const float* in = q + ((long)t * H + h) * hw + d + e;
+    float a = 0.f, b = 0.f;
+    for (int s = 0; s < nsplit; ++s) {
+      a += in[s * split_stride];
+      b += in[s * split_stride + half];
+    }
+    const float cs = cos_t[(long)t * half + e], sn = sin_t[(long)t * half + e];
+    bf16_t* dst = out + t * row_out + (long)h * (rank + dr) + rank + e;
+    dst[0] = (bf16_t)(a * cs - b * sn);
+    dst[half] = (bf16_t)(b * cs + a * sn);
+  }
+  __syncthreads();
+  for (int r0 = 32 * wave; r0 < rank; r0 += 32 * (kLatThreads / kWave)) {
+    const bf16_t* wrow = w_ukt + ((long)h * rank + min(r0 + c, rank - 1)) * d + 8 * g;
+    bf16x8 a[DS];
+#pragma unroll
+    for (int k = 0; k < DS; ++k) a[k] = *reinterpret_cast<const bf16x8*>(wrow + 16 * k);
+#pragma unroll
+    for (int tb = 0; tb < kLatTokens / 32; ++tb) {
+      floatx16 acc = {};
+#pragma unroll
+      for (int k = 0; k < DS; ++k)
+        acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[k], *reinterpret_cast<const bf16x8*>(qs + (32 * tb + c) * LD + 16 * k + 8 * g),
+                                                      acc, 0, 0, 0);
+      const int t = t0 + 32 * tb + c;
+      if (t >= n) continue;
+      bf16_t* dst = out + t * row_out + (long)h * (rank + dr) + r0 + 4 * g;
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+        if (r0 + 8 * b + 4 * g < rank)                        // rank in steps of 4 (the launch)
+          *reinterpret_cast<bf16x4*>(dst + 8 * b) =
+              bf16x4{(bf16_t)acc[4 * b], (bf16_t)acc[4 * b + 1], (bf16_t)acc[4 * b + 2], (bf16_t)acc[4 * b + 3]};
+    }
+  }
+}
+
+// A wave takes 32 outputs and 32 of the tokens, the rank in steps of 16, eight steps' pieces in flight.
+__global__ __launch_bounds__(kLatThreads) void latent_out_block_kernel(
+    const bf16_t* __restrict__ attended, const bf16_t* __restrict__ w_uv, const float* __restrict__ gate, int nsplit,
+    long split_stride, long gate_stride, int by_head, bf16_t* __restrict__ out, int n, int H, int dv, int rank) {
+  constexpr int kAhead = 8;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int g = lane / 32, c = lane % 32;
+  const int h = blockIdx.x, t0 = blockIdx.y * kLatTokens + 32 * (wave % 2);
+  const int j0 = (2 * blockIdx.z + wave / 2) * 32;
+  if (j0 >= dv || t0 >= n) return;
+  const bf16_t* wrow = w_uv + ((long)h * dv + min(j0 + c, dv - 1)) * rank + 8 * g;
+  const bf16_t* arow = attended + ((long)min(t0 + c, n - 1) * H + h) * rank + 8 * g;
+  floatx16 acc = {};
+  const int steps = rank / 16;
+  for (int k0 = 0; k0 < steps; k0 += kAhead) {
+    bf16x8 a[kAhead], b[kAhead];
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k) {
+      const int at = 16 * min(k0 + k, steps - 1);
+      a[k] = *reinterpret_cast<const bf16x8*>(wrow + at);
+      b[k] = *reinterpret_cast<const bf16x8*>(arow + at);
+    }
+#pragma unroll
+    for (int k = 0; k < kAhead; ++k)
+      if (k0 + k < steps) acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[k], b[k], acc, 0, 0, 0);
+  }
+  const int t = t0 + c;
+  if (t >= n) return;
+#pragma unroll
+  for (int b = 0; b < 4; ++b) {
+    const int j = j0 + 8 * b + 4 * g;
+    if (j >= dv) continue;                                    // dv in steps of 4 (the launch)
+    float z[4] = {0.f, 0.f, 0.f, 0.f};
+    if (gate) {
+      const float* at = gate + t * gate_stride + (by_head ? h : (long)h * dv + j);
+      for (int s = 0; s < nsplit; ++s)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) z[e] += at[s * split_stride + (by_head ? 0 : e)];
+    }
+    bf16x4 v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = (bf16_t)(gate ? acc[4 * b + e] * sigmoid_f32(z[e]) : acc[4 * b + e]);
+    *reinterpret_cast<bf16x4*>(out + ((long)t * H + h) * dv + j) = v;
+  }
+}
+
 }  // namespace kllm
 
 using namespace kllm;
@@ -800,12 +1015,18 @@ extern "C" int kllm_latent_norm(const float* in, int nsplit, long split_stride, 
                                 float eps, void* out, int n, int r, int dtype, hipStream_t stream) {
   KLLM_REQUIRE(in && weight && out && n > 0 && r > 0 && nsplit >= 1 && in_stride >= r, "latent_norm: null pointer or bad sizes");
   KLLM_REQUIRE(dtype == DT_F32 || dtype == DT_BF16, "latent_norm: unknown dtype %d", dtype);
-  if (dtype == DT_F32)
-    hipLaunchKernelGGL(latent_norm_kernel<float>, dim3(n), dim3(kLatThreads), 0, stream, in, nsplit, split_stride,
-                       in_stride, weight, eps, (float*)out, r);
-  else
-    hipLaunchKernelGGL(latent_norm_kernel<bf16_t>, dim3(n), dim3(kLatThreads), 0, stream, in, nsplit, split_stride,
-                       in_stride, weight, eps, (bf16_t*)out, r);
+#define KLLM_LN(T, PER)                                                                                              \
+  hipLaunchKernelGGL((latent_norm_kernel<T, PER>), dim3(n), dim3(kLatThreads), 0, stream, in, nsplit, split_stride,  \
+                     in_stride, weight, eps, (T*)out, r)
+#define KLLM_LNS(T)                                                        \
+  do {                                                                     \
+    if (r <= 4 * kLatThreads) KLLM_LN(T, 4);                               \
+    else if (r <= 16 * kLatThreads) KLLM_LN(T, 16);                        \
+    else KLLM_LN(T, 0);                                                    \
+  } while (0)
+  if (dtype == DT_F32) KLLM_LNS(float); else KLLM_LNS(bf16_t);
+#undef KLLM_LNS
+#undef KLLM_LN
   KLLM_CHECK_LAUNCH("latent_norm");
   return 0;
 }
@@ -821,6 +1042,18 @@ extern "C" int kllm_latent_query(const float* q, int nsplit, long split_stride, 
   if (transposed) {     // w_uk is [H][rank][d]: the kernel on the matrix cores
     KLLM_REQUIRE(dtype == DT_BF16 && d % 32 == 0 && ((uintptr_t)w_uk & 15) == 0,
                  "latent_query: the transposed matrix goes with bfloat16 and head sizes in steps of 32 (d=%d)", d);
+    if (n >= kLatTokens && rank % 4 == 0 && dr % 4 == 0 && d <= 256 && ((uintptr_t)out & 7) == 0 && (n + kLatTokens - 1) / kLatTokens <= 65535) {
+      const dim3 grid(H, (n + kLatTokens - 1) / kLatTokens);
+#define KLLM_LQ(DS)                                                                                                   \
+  case DS / 2:                                                                                                        \
+    hipLaunchKernelGGL(latent_query_block_kernel<DS>, grid, dim3(kLatThreads), 0, stream, q, nsplit, split_stride,    \
+                       (const bf16_t*)w_uk, cos_t, sin_t, (bf16_t*)out, n, H, dr, rank);                              \
+    break
+      switch (d / 32) { KLLM_LQ(2); KLLM_LQ(4); KLLM_LQ(6); KLLM_LQ(8); KLLM_LQ(10); KLLM_LQ(12); KLLM_LQ(14); KLLM_LQ(16); }
+#undef KLLM_LQ
+      KLLM_CHECK_LAUNCH("latent_query");
+      return 0;
+    }
     hipLaunchKernelGGL(latent_query_mfma_kernel, dim3((n + 15) / 16, H, (rank + 63) / 64), dim3(kLatThreads), 0, stream, q,
                        nsplit, split_stride, (const bf16_t*)w_uk, cos_t, sin_t, (bf16_t*)out, n, H, d, dr, rank);
     KLLM_CHECK_LAUNCH("latent_query");
@@ -881,6 +1114,14 @@ extern "C" int kllm_latent_out(const void* attended, const void* w_uv, const flo
   KLLM_REQUIRE(n > 0 && H > 0 && H <= 65535 && dv > 0 && rank > 0 && rank <= 8192 && (!gate || nsplit >= 1),
                "latent_out: bad sizes n=%d H=%d dv=%d rank=%d", n, H, dv, rank);
   KLLM_REQUIRE(dtype == DT_F32 || dtype == DT_BF16, "latent_out: unknown dtype %d", dtype);
+  if (dtype == DT_BF16 && n >= kLatTokens && rank % 16 == 0 && dv % 4 == 0 && ((uintptr_t)attended & 15) == 0 &&
+      ((uintptr_t)w_uv & 15) == 0 && ((uintptr_t)out & 7) == 0 && (n + kLatTokens - 1) / kLatTokens <= 65535) {
+    hipLaunchKernelGGL(latent_out_block_kernel, dim3(H, (n + kLatTokens - 1) / kLatTokens, (dv + 63) / 64), dim3(kLatThreads), 0,
+                       stream, (const bf16_t*)attended, (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride,
+                       gate_by_head, (bf16_t*)out, n, H, dv, rank);
+    KLLM_CHECK_LAUNCH("latent_out");
+    return 0;
+  }
   if (dtype == DT_BF16 && rank % 32 == 0 && ((uintptr_t)attended & 15) == 0 && ((uintptr_t)w_uv & 15) == 0) {
     hipLaunchKernelGGL(latent_out_mfma_kernel, dim3((n + 15) / 16, H, (dv + 63) / 64), dim3(kLatThreads), 0, stream,
                        (const bf16_t*)attended, (const bf16_t*)w_uv, gate, nsplit, split_stride, gate_stride, gate_by_head,
