@@ -475,7 +475,7 @@ template <int NR, int KS>
 __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
     const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
     const int* __restrict__ positions, const int* __restrict__ span_of_token, const int* __restrict__ block_table,
-    int max_pages, int page_size, unsigned page_magic, int n, int H, int row, int rank, float scale, int window) {
+    int max_pages, int page_size, unsigned page_magic, int n, int H, int row, int rank, float scale, int window, int redo) {
   extern __shared__ __attribute__((aligned(16))) bf16_t lat_tiles[];
   // page of a key without a division: page_magic = ceil(2^35 / page_size) from the host, exact for
   // keys below 2^24 and pages of up to 2,048 slots (checked at the launch)
@@ -491,6 +491,8 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
   const bool token_ok = t_first + wave < n;
   const int head = min(h0 + c, H - 1);
   const bool head_ok = h0 + c < H;
+  // behind attn_latent_columns_kernel: only where that left a column to be done
+  if (redo && !__syncthreads_or(token_ok && head_ok && isnan((float)out[((long)t * H + head) * rank]))) return;
   const int my_span = span_of_token[t];
   const int len = positions[t] + 1;
   const int lo = first_key(len - 1, window, 0);
@@ -691,6 +693,275 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_block_kernel(
   }
 }
 
+// The same for long steps of the common sizes (rank and rows in steps of 32): the (token, head) pairs of a
+// step in a row are columns, 128 to a workgroup and 32 to a wave, and the products are MFMA 32x32x16
+// (lane l: g = l/32, c = l%32: A[c][8g..8g+7], B[8g..8g+7][c], D[8(i/4) + 4g + i%4][c]).  Scores S^T =
+// K Q^T: A = 32 keys x 16 of their rows from LDS, B = the columns' folded queries, which stay in
+// registers; a lane holds 16 scores of one column, lane ^ 32 the other 16.  Weighted sum O^T += C^T P^T:
+// the 16 slots of MFMA u are the keys 16u + 8(j/4) + 4g + j%4, j = 0..7, which are the scores 8u + j a
+// lane holds; A = latents [element c][those keys], two 8-byte reads.
+//
+// A tile of 32 keys (rows, then latents with the keys side by side) goes from the pages straight into one of
+// two LDS buffers (global loads that write LDS: 16 bytes a lane, a wave's 64 pieces in a row), the
+// next tile's while this one is multiplied.  A wave cannot pad what it writes this way, so the 16-byte
+// pieces of a row change places: piece p of key row k lies at p ^ (k & row_mask), piece p of
+// element e's 32 keys at p ^ (e/4 % 4), which spreads a read over the banks.
+//
+// The accumulators fill the matrix unit's own registers, and the query's pieces most of the others: there
+// is no room to bring an output to a new maximum.  Probabilities are taken relative to the largest score
+// of the column's first tile instead, which is exact as long as no later score is more than kLatRange
+// binary orders above it (32-bit and bfloat16 numbers have the same exponents, and what they hold relative to
+// the largest is the same).  A column where one is leaves a NaN as its first element, and the launch
+// behind this one (attn_latent_block_kernel, which otherwise ends at once) takes its place.
+constexpr int kLatColumns = 128;      // of a workgroup
+constexpr float kLatRange = 60.f;
+
+__device__ __forceinline__ unsigned lds_address(const void* p) {
+  return (unsigned)(size_t)(__attribute__((address_space(3))) const void*)p;
+}
+// 16 bytes a lane from base + offset (base, lds the same in every lane) to lds + 16 * lane.
+__device__ __forceinline__ void load_to_lds(unsigned lds, const void* base, unsigned offset) {
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2" ::"s"(lds), "v"(offset), "s"(base) : "memory", "m0");
+}
+// The same from an address of the lane's own.
+__device__ __forceinline__ void load_to_lds(unsigned lds, const void* address) {
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(lds), "v"(address) : "memory", "m0");
+}
+
+template <int NB, int KS>   // latents of 32 NB elements, rows of 16 KS
+__global__ __launch_bounds__(64 * kLatWaves) __attribute__((amdgpu_waves_per_eu(NB <= 4 ? 2 : 1))) void attn_latent_columns_kernel(
+    const bf16_t* __restrict__ q, bf16_t* __restrict__ out, const bf16_t* __restrict__ cache,
+    const int* __restrict__ positions, const int* __restrict__ span_of_token, const int* __restrict__ block_table,
+    int max_pages, int page_size, unsigned page_magic, int n, int H, float scale, int window) {
+  constexpr int rank = 32 * NB, row = 16 * KS, row8 = row / 8;
+  constexpr int row_mask = row8 % 8 == 0 ? 7 : row8 % 4 == 0 ? 3 : 1;
+  extern __shared__ __attribute__((aligned(16))) bf16_t lat_tiles[];   // two buffers: [32][row], [rank][32]
+  auto page_index = [&](int key) { return (int)(__umulhi((unsigned)key, page_magic) >> 3); };
+  const int tid = threadIdx.x, lane = tid % kWave, wave = __builtin_amdgcn_readfirstlane(tid / kWave);
+  const int g = lane / 32, c = lane % 32;
+  constexpr int buf_elems = 32 * row + 32 * rank;
+  // later tokens of a prompt read more keys: the workgroups with the most to do start first
+  const long col0 = (long)(gridDim.x - 1 - blockIdx.x) * kLatColumns;
+  const long ncols = (long)n * H;
+  const int t_first = (int)(col0 / H), t_last = (int)((min(col0 + kLatColumns, ncols) - 1) / H);
+  const long col = min(col0 + 32 * wave + c, ncols - 1);
+  const bool col_ok = col0 + 32 * wave + c < ncols;
+  const int t = (int)(col / H);
+  const int my_span = span_of_token[t];
+  const int len = positions[t] + 1;
+  const int lo = first_key(len - 1, window, 0);
+  const long page_elems = (long)page_size * (row + rank);
+  const float c2 = scale * 1.4426950408889634f;             // scale * log2(e)
+  bf16x8 qreg[KS];
+#pragma unroll
+  for (int kk = 0; kk < KS; ++kk) qreg[kk] = *reinterpret_cast<const bf16x8*>(q + col * row + 16 * kk + 8 * g);
+
+  float m = -INFINITY, l = 0.f;
+  floatx16 acc[NB];
+#pragma unroll
+  for (int r = 0; r < NB; ++r)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) acc[r][i] = 0.f;
+
+  // ---- where this lane's pieces of a tile come from.  Rows: load j of the wave (every fourth one) fills the
+  // 64 pieces from 64 (4 j + wave) on; a half (16 keys, 2 row8 whole loads) lies in one page.  Latents:
+  // load j fills 16 elements' pieces; the lane's piece, and with it its half, is the same in all of them.
+  constexpr int KL = KS / 4 + (KS % 4 ? 1 : 0);              // loads of a wave: 32 rows of 2 KS pieces over 256 lanes
+  unsigned k_off[KL];
+#pragma unroll
+  for (int j = 0; j < KL; ++j) {
+    const int piece = 64 * (4 * j + wave) + lane;
+    const int kr = piece / row8, kp = piece - kr * row8;
+    k_off[j] = (unsigned)(((kr % 16) * row + 8 * (kp ^ (kr & row_mask))) * (int)sizeof(bf16_t));
+  }
+  const int v_piece = (lane % 4) ^ (lane / 16 % 4), v_half = v_piece / 2;
+  const unsigned lds0 = lds_address(lat_tiles);
+  // ... and where it reads them: four places each, the rest are constant distances
+  int k_at[4], v_at[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    k_at[j] = c * row + 8 * ((2 * j + g) ^ (c & row_mask));
+    v_at[j] = c * 32 + 8 * (j ^ (c / 4 % 4)) + 4 * g;
+  }
+
+  bool over = false;
+  for (int first = t_first; first <= t_last;) {
+    const int span = span_of_token[first];
+    int last = first;
+    while (last < t_last && span_of_token[last + 1] == span) ++last;
+    const int group_len = positions[last] + 1;                // the span's last token here reads the most keys
+    const int group_lo = first_key(positions[first], window, 0);   // ... and its first the earliest (pages before it may be gone)
+    const bool mine = col_ok && my_span == span;
+    const int* table = block_table + (long)span * max_pages;
+    auto half_live = [&](int k0) { return k0 < group_len && k0 + 16 > group_lo; };
+    struct Halves {
+      int page[2];
+    };
+    // a vector load although the address is the same in every lane (see fetch: it has the loop's turn to arrive)
+    auto lookup = [&](int kb) -> Halves {
+      Halves P;
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        int index = half_live(kb + 16 * u) ? page_index(kb + 16 * u) : 0;
+        asm volatile("" : "+v"(index));
+        P.page[u] = table[index];
+      }
+      return P;
+    };
+    auto fetch = [&](int kb, const Halves& P, int buf) {
+      const bf16_t* base[2];
+      int slot[2];
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const int k0 = kb + 16 * u;
+        const bool live = half_live(k0);                      // a half that nobody reads takes page 0
+        const int page = __builtin_amdgcn_readfirstlane(P.page[u]);
+        base[u] = cache + (long)(live ? page : 0) * page_elems;
+        slot[u] = live ? k0 - page_index(k0) * page_size : 0;
+      }
+      const unsigned k_lds = lds0 + (unsigned)(buf * buf_elems) * (unsigned)sizeof(bf16_t);
+      const unsigned v_lds = k_lds + (unsigned)(32 * row) * (unsigned)sizeof(bf16_t);
+#pragma unroll
+      for (int j = 0; j < KL; ++j) {
+        const int load = 4 * j + wave;                        // of KS
+        if (load >= KS) continue;
+        const int u = 2 * load >= KS;                         // the first KS / 2 loads are the first half's
+        load_to_lds(k_lds + 1024u * (unsigned)load, u ? base[1] + (long)slot[1] * row : base[0] + (long)slot[0] * row, k_off[j]);
+      }
+      const bf16_t* v0 = base[0] + (long)page_size * row + slot[0];
+      const bf16_t* v1 = base[1] + (long)page_size * row + slot[1];
+      const bf16_t* vsrc = (v_half ? v1 : v0) + 8 * (v_piece % 2) + (long)(lane / 4) * page_size;
+#pragma unroll
+      for (int j = 0; j < NB / 2; ++j) {
+        const int load = 4 * j + wave;                        // of 2 NB
+        load_to_lds(v_lds + 1024u * (unsigned)load, vsrc + (long)(16 * load) * page_size);
+      }
+    };
+    const int kb0 = group_lo / 32 * 32;
+    Halves pages = lookup(kb0);
+    __syncthreads();                                          // the span before this one has been worked through
+    fetch(kb0, pages, 0);
+    pages = lookup(kb0 + 32);
+    int buf = 0;
+    for (int kb = kb0; kb < group_len; kb += 32, buf ^= 1) {
+      asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");   // this wave's part of the tile is in LDS, its reads of the last one are done
+      __builtin_amdgcn_s_barrier();
+      asm volatile("" ::: "memory");
+      if (kb + 32 < group_len) {                              // (the same for all)
+        fetch(kb + 32, pages, buf ^ 1);
+        pages = lookup(kb + 64);
+      }
+      bf16_t* const ks = lat_tiles + buf * buf_elems;         // [32][row]
+      bf16_t* const vs = ks + 32 * row;                       // [rank][32]
+      if (kb + 32 > group_len || !half_live(kb)) {            // latents of slots that may hold anything become zeros
+        for (int i = tid; i < 32 * rank; i += 64 * kLatWaves) {
+          const int key = kb + i % 32;
+          if (key >= group_len || !half_live(kb + i % 32 / 16 * 16)) {
+            const int e = i / 32, piece = i % 32 / 8;
+            vs[e * 32 + 8 * (piece ^ (e / 4 % 4)) + i % 8] = (bf16_t)0.f;
+          }
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+      }
+      if (!__any(mine && kb < len && kb + 32 > lo)) continue;
+      // ---- scores: this lane's key row is c
+      // (a group of pieces is read while the one before it is multiplied, and no more: registers)
+      constexpr int kGroup = 2;
+      floatx16 s0 = {}, s1 = {};
+      bf16x8 ka[2][kGroup];
+#pragma unroll
+      for (int j = 0; j < kGroup; ++j) ka[0][j] = *reinterpret_cast<const bf16x8*>(ks + k_at[j]);
+#pragma unroll
+      for (int k0 = 0; k0 < KS; k0 += kGroup) {               // piece 2 kk + g of the row, at its swapped place
+#pragma unroll
+        for (int j = 0; j < kGroup; ++j) {
+          const int kk = k0 + kGroup + j;
+          if (kk < KS) ka[(k0 / kGroup + 1) % 2][j] = *reinterpret_cast<const bf16x8*>(ks + k_at[kk % 4] + 64 * (kk / 4));
+        }
+        __builtin_amdgcn_sched_barrier(0);
+        s0 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka[k0 / kGroup % 2][0], qreg[k0], s0, 0, 0, 0);
+        s1 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ka[k0 / kGroup % 2][1], qreg[k0 + 1], s1, 0, 0, 0);
+        __builtin_amdgcn_sched_barrier(0);
+      }
+      const int hi_e = mine ? len - 1 - kb - 4 * g : -1, lo_e = lo - kb - 4 * g;    // offsets that this lane's column reads
+      float tmax = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int e = 8 * (i / 4) + i % 4;
+        s0[i] = (e <= hi_e && e >= lo_e) ? (s0[i] + s1[i]) * c2 : -INFINITY;
+        tmax = fmaxf(tmax, s0[i]);
+      }
+      tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
+      if (m == -INFINITY) m = tmax;                           // the column's first keys
+      over |= tmax > m + kLatRange;
+      const float mref = m == -INFINITY ? 0.f : m;            // (a column without a key so far: every score is -inf)
+      bf16x8 pb[2];
+      float psum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const bf16_t p = (bf16_t)__builtin_amdgcn_exp2f(s0[i] - mref);      // exp2(-inf) = 0
+        pb[i / 8][i % 8] = p;
+        psum += (float)p;
+      }
+      l += psum;
+      // ---- the weighted sum of the latents
+      {
+        bf16x4 va[2][4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) va[0][j] = *reinterpret_cast<const bf16x4*>(vs + v_at[j]);
+#pragma unroll
+        for (int r = 0; r < NB; ++r) {
+          if (r + 1 < NB)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) va[(r + 1) % 2][j] = *reinterpret_cast<const bf16x4*>(vs + v_at[j] + 1024 * (r + 1));
+          __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            const bf16x4 a0 = va[r % 2][2 * u], a1 = va[r % 2][2 * u + 1];
+            const bf16x8 a = {a0[0], a0[1], a0[2], a0[3], a1[0], a1[1], a1[2], a1[3]};
+            acc[r] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, pb[u], acc[r], 0, 0, 0);
+          }
+          __builtin_amdgcn_sched_barrier(0);
+        }
+      }
+    }
+    first = last + 1;
+  }
+  l += __shfl_xor(l, 32, kWave);
+  if (!col_ok) return;
+  const float inv = over ? NAN : 1.f / l;
+  bf16_t* orow = out + col * rank;
+#pragma unroll
+  for (int r = 0; r < NB; ++r)
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+      bf16x4 v;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = (bf16_t)(acc[r][4 * b + i] * inv);
+      *reinterpret_cast<bf16x4*>(orow + 32 * r + 8 * b + 4 * g) = v;
+    }
+}
+
+template <int NB, int KS>
+static int launch_latent_columns(const void* q, void* out, const void* cache, const int* positions, const int* span_of_token,
+                                 const int* block_table, int max_pages, int page_size, int n, int H, float scale, int window,
+                                 hipStream_t stream) {
+  const size_t lds = 2 * (size_t)(32 * 16 * KS + 32 * 32 * NB) * sizeof(bf16_t);
+  static size_t raised_to = 64 * 1024;
+  if (lds > raised_to) {
+    hipError_t e = hipFuncSetAttribute((const void*)attn_latent_columns_kernel<NB, KS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) KLLM_FAIL((int)e, "attn_latent: cannot raise the LDS limit: %s", hipGetErrorString(e));
+    raised_to = lds;
+  }
+  const unsigned page_magic = (unsigned)(((1ull << 35) + page_size - 1) / page_size);
+  hipLaunchKernelGGL((attn_latent_columns_kernel<NB, KS>), dim3(ceil_div((long)n * H, kLatColumns)), dim3(64 * kLatWaves), lds, stream,
+                     (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, span_of_token, block_table, max_pages,
+                     page_size, page_magic, n, H, scale, window);
+  return 0;
+}
+
 // The slices' results of one (token, head) become its output: weights exp(m_s - max m).  A lane takes one
 // slice's maximum and sum (up to 64 slices) and works out its weight; the weights wait in LDS while
 // eight slices' outputs at a time are asked for.
@@ -726,7 +997,7 @@ __global__ __launch_bounds__(kLatThreads) void attn_latent_merge_kernel(const fl
 template <int NR, int KS>
 static void launch_latent_mfma(const void* q, void* out, const void* cache, const int* positions, const int* span_of_token,
                                const int* block_table, int max_pages, int page_size, int n, int H, int row, int rank,
-                               float scale, int window, float* part, int nslices, hipStream_t stream) {
+                               float scale, int window, float* part, int nslices, int redo, hipStream_t stream) {
   const size_t lds = (size_t)(kLatWaves - 1) * (NR * 4 + 2) * kWave * sizeof(float);
   const unsigned page_magic = (unsigned)(((1ull << 35) + page_size - 1) / page_size);
   static int raised = 0;
@@ -743,7 +1014,7 @@ static void launch_latent_mfma(const void* q, void* out, const void* cache, cons
     }
     hipLaunchKernelGGL((attn_latent_block_kernel<NR, KS>), dim3((n + kLatWaves - 1) / kLatWaves, (H + 15) / 16), dim3(64 * kLatWaves),
                        tiles, stream, (const bf16_t*)q, (bf16_t*)out, (const bf16_t*)cache, positions, span_of_token,
-                       block_table, max_pages, page_size, page_magic, n, H, row, rank, scale, window);
+                       block_table, max_pages, page_size, page_magic, n, H, row, rank, scale, window, redo);
     return;
   }
   hipLaunchKernelGGL((attn_latent_mfma_kernel<NR, KS>), dim3(n, (H + 15) / 16, nslices), dim3(64 * kLatWaves), lds, stream,
@@ -1085,9 +1356,23 @@ extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, con
     KLLM_REQUIRE(nslices >= 0 && nslices <= 64 && (nslices <= 1 || (part && part_floats >= (long)n * H * nslices * (rank + 2))),
                  "attn_latent: %d slices need room for %d tokens x %d heads x %d slices x (%d + 2) floats", nslices, n, H,
                  nslices, rank);
+    int redo = 0;
+    if (nslices == 0 && (long)n * H / kLatColumns < (1L << 30)) {
+      // the sizes that are built for long steps: (rank, row) = 32 NB, 16 KS
+#define KLLM_LATC(NB, KS)                                                                                               \
+  if (rank == 32 * NB && row == 16 * KS) {                                                                              \
+    if (int rc = launch_latent_columns<NB, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, \
+                                               H, scale, window, stream))                                               \
+      return rc;                                                                                                        \
+    redo = 1;                                                                                                           \
+  }
+      KLLM_LATC(2, 6) KLLM_LATC(2, 8) KLLM_LATC(4, 10) KLLM_LATC(4, 12) KLLM_LATC(8, 18) KLLM_LATC(8, 20) KLLM_LATC(16, 34)
+      KLLM_LATC(16, 36)
+#undef KLLM_LATC
+    }
     // the latent's accumulators and the query's pieces in registers: built for ranks up to 128, 256 and
     // 512 with rows of up to 256, 384 and 640; longer rows ask for the query at every tile
-#define KLLM_LAT(NR, KS) launch_latent_mfma<NR, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, H, row, rank, scale, window, part, nslices, stream)
+#define KLLM_LAT(NR, KS) launch_latent_mfma<NR, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, H, row, rank, scale, window, part, nslices, redo, stream)
     if (rank <= 128) { if (row <= 256) KLLM_LAT(8, 8); else KLLM_LAT(8, 0); }
     else if (rank <= 256) { if (row <= 384) KLLM_LAT(16, 12); else KLLM_LAT(16, 0); }
     else { if (row <= 640) KLLM_LAT(32, 20); else KLLM_LAT(32, 0); }
