@@ -243,7 +243,7 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     const int* __restrict__ positions, const int* __restrict__ span_of_token, const int* __restrict__ block_table,
     int max_pages, int page_size, unsigned page_magic, int H, int row, int rank, float scale, int window,
     float* __restrict__ part) {
-  extern __shared__ float lat_red[];            // [kLatWaves - 1][NR * 4 + 2][64]
+  extern __shared__ float lat_red[];            // [kLatWaves][NR * 4 + 2][64]
   const int lane = threadIdx.x % kWave, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
   const int g = lane / 16, c = lane % 16;
   const int t = blockIdx.x, h0 = blockIdx.y * 16;
@@ -293,44 +293,48 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     }
     const bf16_t* krow[2] = {pbase[0] + (long)slot0[0] * row, pbase[1] + (long)slot0[1] * row};      // + this lane's place
     const bf16_t* vt[2] = {pbase[0] + (long)page_size * row + slot0[0], pbase[1] + (long)page_size * row + slot0[1]};
-    // ---- the latents' pieces, RB at a time: the first are asked for before the scores are worked on
-    constexpr int RB = 8;
+    // ---- the latents' pieces, RB at a time: the first asked for behind the scores' products
+    constexpr int RB = NR < 16 ? NR : 16;
     struct Piece {
       bf16x4 v[RB][2];
     };
     auto v_fetch = [&](int r0) -> Piece {
       Piece P;
 #pragma unroll
-      for (int j = 0; j < RB; ++j)
+      for (int r = 0; r < RB; ++r)
 #pragma unroll
         for (int u = 0; u < 2; ++u)
-          P.v[j][u] = *reinterpret_cast<const bf16x4*>(vt[u] + (long)(16 * min(r0 + j, nr - 1)) * page_size + v_lane);
+          P.v[r][u] = *reinterpret_cast<const bf16x4*>(vt[u] + (long)(16 * min(r0 + r, nr - 1)) * page_size + v_lane);
       return P;
     };
     floatx4 s[2] = {floatx4{0.f, 0.f, 0.f, 0.f}, floatx4{0.f, 0.f, 0.f, 0.f}};
-    Piece piece;
     if constexpr (KS > 0) {
-      constexpr int KB = KS % 6 == 0 ? 6 : KS % 5 == 0 ? 5 : 4;   // steps whose pieces of the keys are asked for together
+      // the keys' pieces, KB steps at a time and one group ahead of the products
+      constexpr int KB = KS % 6 == 0 ? 6 : KS % 5 == 0 ? 5 : 4;
       static_assert(KS % KB == 0, "whole groups of steps");
-#pragma unroll
-      for (int k0 = 0; k0 < KS; k0 += KB) {
-        bf16x8 a[KB][2];
-#pragma unroll
-        for (int j = 0; j < KB; ++j)
-#pragma unroll
-          for (int u = 0; u < 2; ++u) {
-            const int d0 = 32 * (k0 + j) + 8 * g;
-            a[j][u] = *reinterpret_cast<const bf16x8*>(krow[u] + k_lane + (unsigned)(d0 < row ? 32 * (k0 + j) : 0));
-          }
-        if (k0 + KB >= KS) piece = v_fetch(0);
-        __builtin_amdgcn_sched_barrier(0);                   // (two groups in flight at most: registers)
+      bf16x8 a[2][KB][2];
+      auto k_fetch = [&](bf16x8 (&dst)[KB][2], int j0) {
 #pragma unroll
         for (int j = 0; j < KB; ++j)
 #pragma unroll
           for (int u = 0; u < 2; ++u) {
-            const bool in = 32 * (k0 + j) + 8 * g < row;     // beyond a row: another slot's, anything
-            s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(in ? a[j][u] : zero8, qreg[k0 + j], s[u], 0, 0, 0);
+            const int d0 = 32 * (j0 + j) + 8 * g;
+            dst[j][u] = *reinterpret_cast<const bf16x8*>(krow[u] + k_lane + (unsigned)(d0 < row ? 32 * (j0 + j) : 0));
           }
+      };
+      k_fetch(a[0], 0);
+#pragma unroll
+      for (int j0 = 0; j0 < KS; j0 += KB) {
+        if (j0 + KB < KS) k_fetch(a[(j0 / KB + 1) % 2], j0 + KB);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int j = 0; j < KB; ++j)
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            const bool in = 32 * (j0 + j) + 8 * g < row;     // beyond a row: another slot's, anything
+            s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(in ? a[j0 / KB % 2][j][u] : zero8, qreg[j0 + j], s[u], 0, 0, 0);
+          }
+        __builtin_amdgcn_sched_barrier(0);
       }
     } else {
       for (int ks = 0; ks < ksteps; ++ks) {
@@ -343,8 +347,9 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
           s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(d0 < row ? a : zero8, qb, s[u], 0, 0, 0);
         }
       }
-      piece = v_fetch(0);
     }
+    Piece piece = v_fetch(0);
+    __builtin_amdgcn_sched_barrier(0);
     // ---- online softmax for this lane's head over its 8 keys, then over the 4 lanes of the column
     float tmax = -INFINITY;
 #pragma unroll
@@ -375,94 +380,71 @@ __global__ __launch_bounds__(64 * kLatWaves) void attn_latent_mfma_kernel(
     // ---- the weighted sum of the latents: slots beyond the last key may hold anything
     const bool edge = !live[0] || kb + 32 > len;
 #pragma unroll
-    for (int r0 = 0; r0 < NR; r0 += RB) {
-      const Piece now = piece;
-      if (r0 + RB < NR) piece = v_fetch(r0 + RB);
-      __builtin_amdgcn_sched_barrier(0);
+    for (int r = 0; r < NR; ++r) {
+      if (r < nr) {
+        acc[r] *= alpha;
+        bf16x8 a;
 #pragma unroll
-      for (int j = 0; j < RB; ++j) {
-        const int r = r0 + j;
-        if (r < nr) {
-          acc[r] *= alpha;
-          bf16x8 a;
+        for (int u = 0; u < 2; ++u)
 #pragma unroll
-          for (int u = 0; u < 2; ++u)
-#pragma unroll
-            for (int i = 0; i < 4; ++i)
-              a[4 * u + i] = (!edge || (live[u] && kb + 16 * u + 4 * g + i < len)) ? now.v[j][u][i] : (bf16_t)0.f;
-          acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, acc[r], 0, 0, 0);
-        }
+          for (int i = 0; i < 4; ++i)
+            a[4 * u + i] = (!edge || (live[u] && kb + 16 * u + 4 * g + i < len)) ? piece.v[r % RB][u][i] : (bf16_t)0.f;
+        acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, pb, acc[r], 0, 0, 0);
+      }
+      if (r % RB == RB - 1 && r + 1 < NR) {
+        piece = v_fetch(r + 1);
+        __builtin_amdgcn_sched_barrier(0);
       }
     }
   }
   l += __shfl_xor(l, 16, kWave);
   l += __shfl_xor(l, 32, kWave);
 
-  // ---- the waves meet: waves 1.. leave maximum, sum and output in LDS (lane-contiguous), wave 0
-  // adds them in a fixed order with weights exp(m_w - max m) and writes.
+  // ---- the waves meet: each leaves maximum, sum and output in LDS (lane-contiguous), then adds its share
+  // of the elements of all of them in a fixed order with weights exp(m_w - max m) and writes
   constexpr int kRows = NR * 4 + 2;
-  if (wave > 0) {
-    float* mine = lat_red + (long)(wave - 1) * kRows * kWave + lane;
+  float* mine = lat_red + (long)wave * kRows * kWave + lane;
 #pragma unroll
-    for (int r = 0; r < NR; ++r)
+  for (int r = 0; r < NR; ++r)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) mine[(4 * r + i) * kWave] = acc[r][i];
-    mine[(NR * 4) * kWave] = m;
-    mine[(NR * 4 + 1) * kWave] = l;
-  }
+    for (int i = 0; i < 4; ++i) mine[(4 * r + i) * kWave] = acc[r][i];
+  mine[(NR * 4) * kWave] = m;
+  mine[(NR * 4 + 1) * kWave] = l;
   __syncthreads();
-  if (wave > 0 || !head_ok) return;
-  float mw[kLatWaves - 1], ww[kLatWaves - 1], M = m;
+  if (!head_ok) return;
+  const float* all = lat_red + lane;
+  float ww[kLatWaves], M = -INFINITY, L = 0.f;
 #pragma unroll
-  for (int w = 0; w < kLatWaves - 1; ++w) {
-    mw[w] = lat_red[((long)w * kRows + NR * 4) * kWave + lane];
-    M = fmaxf(M, mw[w]);
+  for (int w = 0; w < kLatWaves; ++w) M = fmaxf(M, all[(w * kRows + NR * 4) * kWave]);
+#pragma unroll
+  for (int w = 0; w < kLatWaves; ++w) {
+    const float mw = all[(w * kRows + NR * 4) * kWave];
+    ww[w] = (mw == -INFINITY) ? 0.f : expf(mw - M);        // (a slice beyond the token's keys has none)
+    L += ww[w] * all[(w * kRows + NR * 4 + 1) * kWave];
   }
-  const float w0 = (m == -INFINITY) ? 0.f : expf(m - M);    // (a slice beyond the token's keys has none)
-  l *= w0;
-#pragma unroll
-  for (int w = 0; w < kLatWaves - 1; ++w) {
-    ww[w] = (mw[w] == -INFINITY) ? 0.f : expf(mw[w] - M);
-    l += ww[w] * lat_red[((long)w * kRows + NR * 4 + 1) * kWave + lane];
-  }
-  if (nslices > 1) {
-    // the slice's sums as they are, with its maximum and its sum of probabilities: rows of
-    // rank + 2 floats; a slice without a key leaves a maximum of -inf and zeros
-    float* prow = part + (((long)t * H + head) * nslices + slice) * (rank + 2);
-#pragma unroll
-    for (int r = 0; r < NR; ++r) {
-      if (r < nr) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float o = acc[r][i] * w0;
-#pragma unroll
-          for (int w = 0; w < kLatWaves - 1; ++w) o += ww[w] * lat_red[((long)w * kRows + 4 * r + i) * kWave + lane];
-          prow[16 * r + 4 * g + i] = o;
-        }
-      }
-    }
-    if (g == 0) {
-      prow[rank] = M;
-      prow[rank + 1] = l;
-    }
-    return;
-  }
-  const float inv = 1.f / l;
+  // of a slice the sums as they are, with its maximum and its sum of probabilities: rows of rank + 2
+  // floats; a slice without a key leaves a maximum of -inf and zeros
+  float* prow = nslices > 1 ? part + (((long)t * H + head) * nslices + slice) * (rank + 2) : nullptr;
+  const float inv = nslices > 1 ? 1.f : 1.f / L;
   bf16_t* orow = out + ((long)t * H + head) * rank;
 #pragma unroll
-  for (int r = 0; r < NR; ++r) {
-    if (r < nr) {
-      bf16x4 v;
+  for (int j = 0; j < NR / kLatWaves; ++j) {
+    const int r = wave * (NR / kLatWaves) + j;
+    if (r >= nr) continue;
+    floatx4 o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        float o = acc[r][i] * w0;
+    for (int w = 0; w < kLatWaves; ++w)
 #pragma unroll
-        for (int w = 0; w < kLatWaves - 1; ++w) o += ww[w] * lat_red[((long)w * kRows + 4 * r + i) * kWave + lane];
-        v[i] = (bf16_t)(o * inv);
-      }
-      *reinterpret_cast<bf16x4*>(orow + 16 * r + 4 * g) = v;
+      for (int i = 0; i < 4; ++i) o[i] = fmaf(ww[w], all[(w * kRows + 4 * r + i) * kWave], o[i]);
+    if (nslices > 1) {                                       // (rows are 8-byte aligned)
+      *reinterpret_cast<floatx2*>(prow + 16 * r + 4 * g) = floatx2{o[0], o[1]};
+      *reinterpret_cast<floatx2*>(prow + 16 * r + 4 * g + 2) = floatx2{o[2], o[3]};
+    } else {
+      *reinterpret_cast<bf16x4*>(orow + 16 * r + 4 * g) =
+          bf16x4{(bf16_t)(o[0] * inv), (bf16_t)(o[1] * inv), (bf16_t)(o[2] * inv), (bf16_t)(o[3] * inv)};
     }
   }
+  if (nslices > 1 && wave == 0 && g == 0) *reinterpret_cast<floatx2*>(prow + rank) = floatx2{M, L};
 }
 
 // The same for steps of many tokens: a workgroup takes four consecutive tokens of the step and up
@@ -998,7 +980,7 @@ template <int NR, int KS>
 static void launch_latent_mfma(const void* q, void* out, const void* cache, const int* positions, const int* span_of_token,
                                const int* block_table, int max_pages, int page_size, int n, int H, int row, int rank,
                                float scale, int window, float* part, int nslices, int redo, hipStream_t stream) {
-  const size_t lds = (size_t)(kLatWaves - 1) * (NR * 4 + 2) * kWave * sizeof(float);
+  const size_t lds = (size_t)kLatWaves * (NR * 4 + 2) * kWave * sizeof(float);
   const unsigned page_magic = (unsigned)(((1ull << 35) + page_size - 1) / page_size);
   static int raised = 0;
   if (lds > 64 * 1024 && !raised) {
@@ -1353,7 +1335,7 @@ extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, con
   if (dtype == DT_BF16 && mode != 1 && rank % 16 == 0 && row % 8 == 0 && rank <= 512 && page_size % 16 == 0 &&
       page_size <= 2048 && (long)max_pages * page_size <= (1L << 24) &&
       ((uintptr_t)q & 15) == 0 && ((uintptr_t)cache & 15) == 0 && ((uintptr_t)out & 7) == 0) {
-    KLLM_REQUIRE(nslices >= 0 && nslices <= 64 && (nslices <= 1 || (part && part_floats >= (long)n * H * nslices * (rank + 2))),
+    KLLM_REQUIRE(nslices >= 0 && nslices <= 64 && (nslices <= 1 || (part && ((uintptr_t)part & 7) == 0 && part_floats >= (long)n * H * nslices * (rank + 2))),
                  "attn_latent: %d slices need room for %d tokens x %d heads x %d slices x (%d + 2) floats", nslices, n, H,
                  nslices, rank);
     int redo = 0;
@@ -1375,7 +1357,7 @@ extern "C" int kllm_attn_latent(const void* q, void* out, const void* cache, con
 #define KLLM_LAT(NR, KS) launch_latent_mfma<NR, KS>(q, out, cache, positions, span_of_token, block_table, max_pages, page_size, n, H, row, rank, scale, window, part, nslices, redo, stream)
     if (rank <= 128) { if (row <= 256) KLLM_LAT(8, 8); else KLLM_LAT(8, 0); }
     else if (rank <= 256) { if (row <= 384) KLLM_LAT(16, 12); else KLLM_LAT(16, 0); }
-    else { if (row <= 640) KLLM_LAT(32, 20); else KLLM_LAT(32, 0); }
+    else { if (row <= 576) KLLM_LAT(32, 18); else if (row <= 640) KLLM_LAT(32, 20); else KLLM_LAT(32, 0); }
 #undef KLLM_LAT
     KLLM_CHECK_LAUNCH("attn_latent");
     return 0;

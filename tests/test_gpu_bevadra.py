@@ -315,7 +315,10 @@ def test_biases_sinks_slopes_window_and_gate_in_the_attention_kernels(H, KV, dk,
 
 
 LATENT_CASES = [(3, 40, 8, 20), (6, 160, 32, 70), (3, 448, 64, 33), (20, 96, 32, 1), (34, 128, 16, 130), (2, 512, 64, 2), (5, 14, 6, 9),
-                (4, 16, 8, 64)]
+                (4, 16, 8, 64),
+                # the sizes whose long steps take 128 (token, head) columns to a workgroup
+                (3, 64, 32, 50), (5, 64, 64, 33), (7, 128, 32, 16), (33, 128, 64, 100), (6, 256, 32, 90), (3, 256, 64, 31),
+                (32, 512, 32, 64), (1, 512, 64, 130)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -379,6 +382,36 @@ def test_latents_behind_a_window(H, rank, dr, window, dtype):
                       page, H, row, rank, scale, plain=plain_kernel, part=part, nslices=slices, window=window)
         got = out.float().cpu().reshape(-1, H, rank)
         assert torch.isfinite(got).all() and rel(got, want[tail]) < tol, (plain_kernel, slices, "pages gone")
+
+
+@pytest.mark.parametrize("H,rank,dr", [(5, 128, 32), (3, 512, 64)])
+def test_scores_that_grow_without_end_through_the_latents(H, rank, dr):
+    """Scores that rise by hundreds from a request's first tile of keys to its last, in one head, and by
+    thousands in another: the kernel of long steps hands such columns on, the others stay."""
+    from kllm_amd import kernels as K
+    page, row, n = 16, rank + dr, 200
+    g = torch.Generator().manual_seed(rank)
+    rows = torch.randn(n, row, generator=g).to(torch.bfloat16)
+    rows[:, 0] = torch.arange(n).float() / n * 4.0
+    cache = torch.full((13, page * (row + rank)), float("nan"))
+    for j in range(13):
+        part = rows[j * page:(j + 1) * page].float()
+        cache[j, :page * row].view(page, row)[:len(part)] = part
+        cache[j, page * row:].view(rank, page)[:, :len(part)] = part[:, :rank].T
+    q = torch.randn(n, H, row, generator=g)
+    q[:, 1, 0], q[150:, 2, 0] = 400.0, 5000.0
+    qd = q.reshape(n, H * row).to(torch.bfloat16)
+    s = torch.einsum("nhd,kd->hnk", qd.double().reshape(n, H, row), rows.double()) * 0.5
+    want = torch.einsum("hnk,kr->nhr", torch.softmax(s.masked_fill(~P.visible(n, 0), float("-inf")), -1), rows[:, :rank].double())
+    assert float(s[1].max()) > 500 and float(s[2].max()) > 5000
+    out = torch.full((n, H * rank), float("nan"), device="cuda", dtype=torch.bfloat16)
+    K.attn_latent(qd.cuda(), out, cache.to("cuda", torch.bfloat16), i32(list(range(n))), i32([0] * n), i32([list(range(13))]), page, H,
+                  row, rank, 0.5, nslices=0)
+    got = out.float().cpu().reshape(n, H, rank)
+    assert torch.isfinite(got).all()
+    for i in range(n):
+        for h in range(H):
+            assert rel(got[i, h], want[i, h]) < 2e-2, (i, h)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
