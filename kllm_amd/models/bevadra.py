@@ -25,7 +25,7 @@ def build_bevadra(cfg: BevadraConfig) -> ModelSpec:
     d = cfg.width
 
     def norm(name):
-        return PartSpec("layernorm", size=d, eps=cfg.norm_eps, names={"weight": name, "bias": name + ".b"})
+        return PartSpec("layer_norm", size=d, eps=cfg.norm_eps, names={"weight": name, "bias": name + ".b"})
 
     positions = {}      # mixers that rotate alike share one position part (and its tables of a step)
 

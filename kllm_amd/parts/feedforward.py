@@ -95,7 +95,8 @@ class GatedFeedForward(Part):
             if normed is not None:
                 return normed
             return linear(ctx, h, self.w_down, "ffn.down")
-        return decode_linear(ctx, h, self.w_down, "ffn.down", self._tiled.get("down"))
+        down = decode_linear(ctx, h, self.w_down, "ffn.down", self._tiled.get("down"))
+        return down if down.dim() == 3 else down[None]         # a stack of sums, also of one
 
 
 @register_part("feed_forward", "dense_mlp")

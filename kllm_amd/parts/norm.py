@@ -122,7 +122,7 @@ class GroupRMSNorm(Part):
         return x
 
 
-@register_part("norm", "layernorm")
+@register_part("norm", "layer_norm")
 class LayerNorm(Part):
     """Layer norm: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b over the channels, in 32-bit.  It
     also adds what is pending to the residual stream: a plain delta, or a ``ScaledSum`` of
